@@ -4,6 +4,7 @@
 // softmax, routing, the residual sum) is fp32 in both.
 //
 //   embed_scale        residual[t] = embed[id[t]] * scale                                (fp32 out)
+//   embed_rmsnorm      residual[t] = rmsnorm(embed[id[t]]) * w                           (fp32 out)
 //   add_rmsnorm        residual += delta;  y = residual * rsqrt(mean(residual^2) + eps) * w
 //   rmsnorm_rows       y = x * rsqrt(mean(x^2) + eps) * w over a column range of a wider row
 //   latent_kv_write    a token's compressed KV entry: RMS-normed latent | rotated shared key part
@@ -14,14 +15,19 @@
 //   sigmoid_gate       y[t, h, :] *= sigmoid(g[t, h])
 //   relu_sq            y = relu(x)^2
 //   glu_clamp          y = g' * sigmoid(alpha g') * (u' + bias),  g' = min(g, limit), u' = clamp(u, +-limit)
+//                      (g and u times a factor of their row first, where one is given)
 //   group_topk         sigmoid scores -> best groups by the sum of their two largest -> top-k experts
 //   route_softmax      softmax scores (+ a selection bias) -> best groups by their largest biased score -> top-k;
 //                      trailing identity experts leave the pair list and come back as one gate per token
 //   rmsnorm_add        residual += rmsnorm(delta) * w;  y = residual (activation dtype)
 //   gated_add_rmsnorm  residual += sigmoid(gate + b) (.) (c1 n1(d1) + c2 n2(d2)) + extra + vector;  y = rmsnorm(residual) w
+//   depth_mix_rmsnorm  s = residual + n(delta) is a layer's result, kept in the history of layer results;
+//                      residual = sum_j a_j history_j + a_last s;  y = rmsnorm(residual) w
+//   poly_norm          y = a N(z) + b N(z^2) + c N(z^3) + e, N = division by the row's root mean square
+//   soft_cap           y = cap tanh(x / cap)                                             (fp32 out)
 //   glu_act            silu(g) * u  or  gelu_tanh(g) * u  of  x = g | u
 //   gather_rows        xs[r] = x[idx[r]]
-//   moe_finish         residual[t] += sum_k w[t,k] * y[pos[t,k]] + gate[t] * shared[t]
+//   moe_finish         residual[t] += sum_k w[t,k] * y[pos[t,k]] + gate[t] * shared[t]   (w optional: all 1)
 //
 // Sizes are free (no multiple-of-8 requirements): these are the plain kernels every shape can take.
 #include "common.h"
@@ -70,6 +76,26 @@ __global__ __launch_bounds__(256) void embed_scale_kernel(const long* __restrict
   const T* e = embed + ids[row] * (long)width;
   float* o = out + row * width;
   for (int i = threadIdx.x; i < width; i += 256) o[i] = Conv<T>::ld(e + i) * scale;
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void embed_rmsnorm_kernel(const long* __restrict__ ids, const T* __restrict__ embed,
+                                                            const float* __restrict__ w, float* __restrict__ out,
+                                                            float* __restrict__ out2, int width, float eps) {
+  __shared__ float red[4];
+  const long row = blockIdx.x;
+  const T* e = embed + ids[row] * (long)width;
+  float ss = 0.f;
+  for (int i = threadIdx.x; i < width; i += 256) {
+    const float v = Conv<T>::ld(e + i);
+    ss += v * v;
+  }
+  const float inv = 1.f / sqrtf(block_sum(ss, red) / (float)width + eps);
+  for (int i = threadIdx.x; i < width; i += 256) {
+    const float v = Conv<T>::ld(e + i) * inv * w[i];
+    out[row * width + i] = v;
+    if (out2) out2[row * width + i] = v;
+  }
 }
 
 // residual fp32 [rows, n] (+= delta, row stride d_stride) -> y (row stride y_stride)
@@ -267,14 +293,16 @@ __global__ __launch_bounds__(256) void relu_sq_kernel(const T* __restrict__ x, T
 
 // x [rows, 2 * inter] (row stride x_stride): gate columns then up columns -> y [rows, inter]
 template <typename T>
-__global__ __launch_bounds__(256) void glu_clamp_kernel(const T* __restrict__ x, long x_stride, T* __restrict__ y,
+__global__ __launch_bounds__(256) void glu_clamp_kernel(const T* __restrict__ x, long x_stride,
+                                                        const float* __restrict__ row_scale, T* __restrict__ y,
                                                         int inter, long total, float limit, float alpha,
                                                         float up_bias) {
   for (long i = blockIdx.x * 256L + threadIdx.x; i < total; i += (long)gridDim.x * 256) {
     const long r = i / inter;
     const int c = (int)(i % inter);
-    const float g = fminf(Conv<T>::ld(x + r * x_stride + c), limit);
-    const float u = fminf(fmaxf(Conv<T>::ld(x + r * x_stride + inter + c), -limit), limit);
+    const float rs = row_scale ? row_scale[r] : 1.f;
+    const float g = fminf(rs * Conv<T>::ld(x + r * x_stride + c), limit);
+    const float u = fminf(fmaxf(rs * Conv<T>::ld(x + r * x_stride + inter + c), -limit), limit);
     Conv<T>::st(y + i, g * sigmoidf(alpha * g) * (u + up_bias));
   }
 }
@@ -588,6 +616,209 @@ __global__ __launch_bounds__(256) void gated_add_rmsnorm_kernel(
   }
 }
 
+// The end of a layer whose result joins a weighted average over the depth.  Per row, with s = residual + n1(delta)
+// (n1(d) = rmsnorm(d) w1 where w1 is given, d itself otherwise; no delta: s = residual):
+//   history[n_prev] = s where `keep`;  residual = sum_{j < n_prev} coef[j] history[j] + coef[n_prev] s;
+//   y = rmsnorm(residual) w
+// history fp32 [*, rows, n], hist_stride elements from one stream to the next.  K as for gated_add_rmsnorm_kernel.
+template <typename T, typename D, int K>
+__global__ __launch_bounds__(256) void depth_mix_rmsnorm_kernel(
+    float* __restrict__ residual, const D* __restrict__ delta, long sd, const float* __restrict__ w1,
+    float* __restrict__ history, long hist_stride, int n_prev, int keep, const float* __restrict__ coef,
+    const float* __restrict__ w, T* __restrict__ y, int n, float eps) {
+  __shared__ float red[4];
+  const long row = blockIdx.x;
+  float* r = residual + row * n;
+  float* hist = history + row * n;
+  const float c_own = coef[n_prev];
+  if constexpr (K > 0) {
+    float x[K][8], d[K][8];
+    float q = 0.f;
+#pragma unroll
+    for (int k = 0; k < K; ++k) {
+      const int i = (threadIdx.x + 256 * k) * 8;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) x[k][e] = d[k][e] = 0.f;
+      if (i < n) {
+        ld8(r + i, x[k]);
+        if (delta) ld8(delta + row * sd + i, d[k]);
+      }
+#pragma unroll
+      for (int e = 0; e < 8; ++e) q += d[k][e] * d[k][e];
+    }
+    float f = 1.f;
+    if (delta && w1) f = 1.f / sqrtf(block_sum(q, red) / (float)n + eps);
+#pragma unroll
+    for (int k = 0; k < K; ++k) {
+      const int i = (threadIdx.x + 256 * k) * 8;
+      if (i < n) {
+        if (delta && w1) {
+          float t[8];
+          ld8(w1 + i, t);
+#pragma unroll
+          for (int e = 0; e < 8; ++e) x[k][e] += d[k][e] * f * t[e];
+        } else {
+#pragma unroll
+          for (int e = 0; e < 8; ++e) x[k][e] += d[k][e];
+        }
+        if (keep) st8(hist + n_prev * hist_stride + i, x[k]);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) x[k][e] *= c_own;
+      }
+    }
+    int j = 0;
+    for (; j + 1 < n_prev; j += 2) {  // two streams' loads in flight
+      const float a0 = coef[j], a1 = coef[j + 1];
+#pragma unroll
+      for (int k = 0; k < K; ++k) {
+        const int i = (threadIdx.x + 256 * k) * 8;
+        if (i < n) {
+          float t[8], u[8];
+          ld8(hist + j * hist_stride + i, t);
+          ld8(hist + (j + 1) * hist_stride + i, u);
+#pragma unroll
+          for (int e = 0; e < 8; ++e) x[k][e] += a0 * t[e] + a1 * u[e];
+        }
+      }
+    }
+    if (j < n_prev) {
+      const float a0 = coef[j];
+#pragma unroll
+      for (int k = 0; k < K; ++k) {
+        const int i = (threadIdx.x + 256 * k) * 8;
+        if (i < n) {
+          float t[8];
+          ld8(hist + j * hist_stride + i, t);
+#pragma unroll
+          for (int e = 0; e < 8; ++e) x[k][e] += a0 * t[e];
+        }
+      }
+    }
+    float ss = 0.f;
+#pragma unroll
+    for (int k = 0; k < K; ++k) {
+      const int i = (threadIdx.x + 256 * k) * 8;
+      if (i < n) st8(r + i, x[k]);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) ss += x[k][e] * x[k][e];
+    }
+    if (!y) return;
+    const float inv = 1.f / sqrtf(block_sum(ss, red) / (float)n + eps);
+#pragma unroll
+    for (int k = 0; k < K; ++k) {
+      const int i = (threadIdx.x + 256 * k) * 8;
+      if (i < n) {
+        float t[8];
+        ld8(w + i, t);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) t[e] *= x[k][e] * inv;
+        st8(y + row * n + i, t);
+      }
+    }
+  } else {
+    float f = 1.f;
+    if (delta && w1) {
+      float q = 0.f;
+      for (int i = threadIdx.x; i < n; i += 256) {
+        const float v = Conv<D>::ld(delta + row * sd + i);
+        q += v * v;
+      }
+      f = 1.f / sqrtf(block_sum(q, red) / (float)n + eps);
+    }
+    float ss = 0.f;
+    for (int i = threadIdx.x; i < n; i += 256) {
+      float v = r[i];
+      if (delta) v += Conv<D>::ld(delta + row * sd + i) * f * (w1 ? w1[i] : 1.f);
+      if (keep) hist[n_prev * hist_stride + i] = v;
+      v *= c_own;
+      for (int j = 0; j < n_prev; ++j) v += coef[j] * hist[j * hist_stride + i];
+      r[i] = v;  // read back below by the same thread
+      ss += v * v;
+    }
+    if (!y) return;
+    const float inv = 1.f / sqrtf(block_sum(ss, red) / (float)n + eps);
+    for (int i = threadIdx.x; i < n; i += 256) Conv<T>::st(y + row * n + i, r[i] * inv * w[i]);
+  }
+}
+
+// Three sums over the workgroup at once
+__device__ __forceinline__ void block_sum3(float& a, float& b, float& c, float (*red)[3]) {
+  a = wave_reduce_sum(a);
+  b = wave_reduce_sum(b);
+  c = wave_reduce_sum(c);
+  const int tid = threadIdx.x;
+  if ((tid & 63) == 0) red[tid >> 6][0] = a, red[tid >> 6][1] = b, red[tid >> 6][2] = c;
+  __syncthreads();
+  a = b = c = 0.f;
+  for (int i = 0; i < (int)(blockDim.x >> 6); ++i) a += red[i][0], b += red[i][1], c += red[i][2];
+}
+
+// y = a N(z) + b N(z^2) + c N(z^3) + e per row, powers element by element, N(v) = v / sqrt(mean(v^2) + eps), the
+// four numbers a, b, c, e in `act`.  K > 0: rows of up to 2048 K values on 16-byte boundaries stay in registers.
+template <typename T, int K>
+__global__ __launch_bounds__(256) void poly_norm_kernel(const T* __restrict__ z, long z_stride,
+                                                        const float* __restrict__ act, T* __restrict__ y, int n,
+                                                        float eps) {
+  __shared__ float red[4][3];
+  const long row = blockIdx.x;
+  const T* zr = z + row * z_stride;
+  T* yr = y + row * n;
+  float s2 = 0.f, s4 = 0.f, s6 = 0.f;
+  if constexpr (K > 0) {
+    float v[K][8];
+#pragma unroll
+    for (int k = 0; k < K; ++k) {
+      const int i = (threadIdx.x + 256 * k) * 8;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) v[k][e] = 0.f;
+      if (i < n) ld8(zr + i, v[k]);
+    }
+#pragma unroll
+    for (int k = 0; k < K; ++k)
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        const float q = v[k][e] * v[k][e];
+        s2 += q;
+        s4 += q * q;
+        s6 += q * q * q;
+      }
+    block_sum3(s2, s4, s6, red);
+    const float a = act[0] / sqrtf(s2 / (float)n + eps), b = act[1] / sqrtf(s4 / (float)n + eps);
+    const float c = act[2] / sqrtf(s6 / (float)n + eps), d = act[3];
+#pragma unroll
+    for (int k = 0; k < K; ++k) {
+      const int i = (threadIdx.x + 256 * k) * 8;
+      if (i < n) {
+        float t[8];
+#pragma unroll
+        for (int e = 0; e < 8; ++e) t[e] = fmaf(v[k][e], fmaf(v[k][e], fmaf(v[k][e], c, b), a), d);
+        st8(yr + i, t);
+      }
+    }
+  } else {
+    for (int i = threadIdx.x; i < n; i += 256) {
+      const float v = Conv<T>::ld(zr + i), q = v * v;
+      s2 += q;
+      s4 += q * q;
+      s6 += q * q * q;
+    }
+    block_sum3(s2, s4, s6, red);
+    const float a = act[0] / sqrtf(s2 / (float)n + eps), b = act[1] / sqrtf(s4 / (float)n + eps);
+    const float c = act[2] / sqrtf(s6 / (float)n + eps), d = act[3];
+    for (int i = threadIdx.x; i < n; i += 256) {
+      const float v = Conv<T>::ld(zr + i);
+      Conv<T>::st(yr + i, fmaf(v, fmaf(v, fmaf(v, c, b), a), d));
+    }
+  }
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void soft_cap_kernel(const T* __restrict__ x, float* __restrict__ y, long n, float cap) {
+  const float inv = 1.f / cap;
+  for (long i = blockIdx.x * 256L + threadIdx.x; i < n; i += (long)gridDim.x * 256)
+    y[i] = cap * tanhf(Conv<T>::ld(x + i) * inv);
+}
+
 // x [rows, 2 inter] = gate | up  ->  act(gate) * up;  kind 0: silu, 1: gelu in its tanh form
 template <typename T>
 __global__ __launch_bounds__(256) void glu_act_kernel(const T* __restrict__ x, long x_stride, T* __restrict__ y,
@@ -628,7 +859,7 @@ __global__ __launch_bounds__(256) void moe_finish_kernel(float* __restrict__ res
   const T* yk[AHEAD];
 #pragma unroll
   for (int k = 0; k < AHEAD; ++k) {
-    wk[k] = k < topk ? weights[t * topk + k] : 0.f;
+    wk[k] = k < topk ? (weights ? weights[t * topk + k] : 1.f) : 0.f;
     yk[k] = y + (long)(wk[k] != 0.f ? pos[t * topk + k] : 0) * n;
   }
   for (int i = threadIdx.x; i < n; i += 256) {
@@ -637,7 +868,7 @@ __global__ __launch_bounds__(256) void moe_finish_kernel(float* __restrict__ res
     for (int k = 0; k < AHEAD; ++k)
       if (wk[k] != 0.f) a += wk[k] * Conv<T>::ld(yk[k] + i);
     for (int k = AHEAD; k < topk; ++k) {
-      const float w = weights[t * topk + k];
+      const float w = weights ? weights[t * topk + k] : 1.f;
       if (w != 0.f) a += w * Conv<T>::ld(y + (long)pos[t * topk + k] * n + i);
     }
     if (shared) a += sg * Conv<T>::ld(shared + t * n + i);
@@ -665,6 +896,16 @@ VPSA_EXPORT int vpsa_embed_scale(const long* ids, const void* embed, float* out,
   DISPATCH(dtype,
            hipLaunchKernelGGL(embed_scale_kernel<bf16_t>, dim3(rows), dim3(256), 0, st, ids, (const bf16_t*)embed, out, width, scale),
            hipLaunchKernelGGL(embed_scale_kernel<float>, dim3(rows), dim3(256), 0, st, ids, (const float*)embed, out, width, scale));
+  return 0;
+}
+
+// out2 (may be null): a second copy of the result
+VPSA_EXPORT int vpsa_embed_rmsnorm(const long* ids, const void* embed, const float* w, float* out, float* out2, int rows,
+                                   int width, float eps, int dtype, hipStream_t st) {
+  if (rows <= 0) return 0;
+  DISPATCH(dtype,
+           hipLaunchKernelGGL(embed_rmsnorm_kernel<bf16_t>, dim3(rows), dim3(256), 0, st, ids, (const bf16_t*)embed, w, out, out2, width, eps),
+           hipLaunchKernelGGL(embed_rmsnorm_kernel<float>, dim3(rows), dim3(256), 0, st, ids, (const float*)embed, w, out, out2, width, eps));
   return 0;
 }
 
@@ -742,13 +983,13 @@ VPSA_EXPORT int vpsa_relu_sq(const void* x, void* y, long n, int dtype, hipStrea
   return 0;
 }
 
-VPSA_EXPORT int vpsa_glu_clamp(const void* x, long x_stride, void* y, int rows, int inter, float limit, float alpha,
+VPSA_EXPORT int vpsa_glu_clamp(const void* x, long x_stride, const float* row_scale, void* y, int rows, int inter, float limit, float alpha,
                                float up_bias, int dtype, hipStream_t st) {
   const long total = (long)rows * inter;
   if (total <= 0) return 0;
   DISPATCH(dtype,
-           hipLaunchKernelGGL(glu_clamp_kernel<bf16_t>, dim3(flat_grid(total)), dim3(256), 0, st, (const bf16_t*)x, x_stride, (bf16_t*)y, inter, total, limit, alpha, up_bias),
-           hipLaunchKernelGGL(glu_clamp_kernel<float>, dim3(flat_grid(total)), dim3(256), 0, st, (const float*)x, x_stride, (float*)y, inter, total, limit, alpha, up_bias));
+           hipLaunchKernelGGL(glu_clamp_kernel<bf16_t>, dim3(flat_grid(total)), dim3(256), 0, st, (const bf16_t*)x, x_stride, row_scale, (bf16_t*)y, inter, total, limit, alpha, up_bias),
+           hipLaunchKernelGGL(glu_clamp_kernel<float>, dim3(flat_grid(total)), dim3(256), 0, st, (const float*)x, x_stride, row_scale, (float*)y, inter, total, limit, alpha, up_bias));
   return 0;
 }
 
@@ -789,6 +1030,60 @@ VPSA_EXPORT int vpsa_gated_add_rmsnorm(float* residual, const void* d1, long s1,
   else { GA(bf16_t, bf16_t); }
 #undef GA
 #undef GA_P
+  return 0;
+}
+
+// d_f32: the delta is fp32 whatever the activation dtype (a mixture's fp32 sum)
+VPSA_EXPORT int vpsa_depth_mix_rmsnorm(float* residual, const void* delta, long sd, int d_f32, const float* w1,
+                                       float* history, long hist_stride, int n_prev, int keep, const float* coef,
+                                       const float* w, void* y, int rows, int n, float eps, int dtype, hipStream_t st) {
+  if (rows <= 0) return 0;
+  if (dtype != 0 && dtype != 1) return -2;
+  if ((y && !w) || !coef || n_prev < 0 || ((n_prev > 0 || keep) && (!history || hist_stride < (long)rows * n))) return -1;
+#define DM_P(T, D, P)                                                                                               \
+  depth_mix_rmsnorm_kernel<T, D, P><<<rows, 256, 0, st>>>(residual, (const D*)delta, sd, w1, history, hist_stride, \
+                                                          n_prev, keep, coef, w, (T*)y, n, eps)
+  auto al = [](const void* p) { return ((uintptr_t)p & 15) == 0; };
+  const bool vec = n % 8 == 0 && sd % 8 == 0 && hist_stride % 4 == 0 && al(residual) && al(delta) && al(w1) &&
+                   al(history) && al(w) && al(y);
+#define DM(T, D)                                 \
+  if (vec && n <= 2048) DM_P(T, D, 1);           \
+  else if (vec && n <= 4096) DM_P(T, D, 2);      \
+  else if (vec && n <= 8192) DM_P(T, D, 4);      \
+  else DM_P(T, D, 0)
+  if (dtype == 1) { DM(float, float); }
+  else if (d_f32) { DM(bf16_t, float); }
+  else { DM(bf16_t, bf16_t); }
+#undef DM
+#undef DM_P
+  return 0;
+}
+
+VPSA_EXPORT int vpsa_poly_norm(const void* z, long z_stride, const float* act, void* y, int rows, int n, float eps,
+                               int dtype, hipStream_t st) {
+  if (rows <= 0) return 0;
+  if (dtype != 0 && dtype != 1) return -2;
+#define PN_P(T, P) poly_norm_kernel<T, P><<<rows, 256, 0, st>>>((const T*)z, z_stride, act, (T*)y, n, eps)
+  const bool vec = n % 8 == 0 && z_stride % 8 == 0 && (((uintptr_t)z | (uintptr_t)y) & 15) == 0;
+#define PN(T)                              \
+  if (vec && n <= 2048) PN_P(T, 1);        \
+  else if (vec && n <= 4096) PN_P(T, 2);   \
+  else if (vec && n <= 8192) PN_P(T, 4);   \
+  else if (vec && n <= 16384) PN_P(T, 8);  \
+  else PN_P(T, 0)
+  if (dtype == 1) { PN(float); }
+  else { PN(bf16_t); }
+#undef PN
+#undef PN_P
+  return 0;
+}
+
+VPSA_EXPORT int vpsa_soft_cap(const void* x, float* y, long n, float cap, int dtype, hipStream_t st) {
+  if (n <= 0) return 0;
+  if (!(cap > 0.f)) return -1;
+  DISPATCH(dtype,
+           hipLaunchKernelGGL(soft_cap_kernel<bf16_t>, dim3(flat_grid(n)), dim3(256), 0, st, (const bf16_t*)x, y, n, cap),
+           hipLaunchKernelGGL(soft_cap_kernel<float>, dim3(flat_grid(n)), dim3(256), 0, st, (const float*)x, y, n, cap));
   return 0;
 }
 

@@ -51,12 +51,14 @@ __global__ __launch_bounds__(256) void moe_topk_softmax_kernel(const uint16_t* _
 }
 
 // Single-workgroup counting sort.  offsets has n_experts + 1 entries; pos[i] is the sorted
-// row of pair i = t*topk + k; sorted_tok[row] = token of that row.  Pairs of one expert keep
+// row of pair i = t*topk + k; sorted_tok[row] = token of that row, sorted_w[row] (optional) its pair's weight.  Pairs of one expert keep
 // their token order (stable), so results do not depend on scheduling.
 __global__ __launch_bounds__(1024) void moe_align_kernel(const int* __restrict__ ids,
                                                          int* __restrict__ offsets,
                                                          int* __restrict__ pos,
-                                                         int* __restrict__ sorted_tok, int n_pairs,
+                                                         int* __restrict__ sorted_tok,
+                                                         const float* __restrict__ weights,
+                                                         float* __restrict__ sorted_w, int n_pairs,
                                                          int n_experts, int topk) {
   __shared__ int cnt[ALIGN_MAX_EXPERTS + 1];
   __shared__ int base[ALIGN_MAX_EXPERTS + 1];
@@ -88,6 +90,7 @@ __global__ __launch_bounds__(1024) void moe_align_kernel(const int* __restrict__
         const int rank = __popcll(m & ((1ull << lane) - 1ull));
         pos[i] = run + rank;
         sorted_tok[run + rank] = i / topk;
+        if (sorted_w) sorted_w[run + rank] = weights[i];
       }
       run += __popcll(m);
     }
@@ -139,10 +142,10 @@ VPSA_EXPORT int vpsa_moe_topk_softmax(const void* logits, float* weights, int* i
 }
 
 VPSA_EXPORT int vpsa_moe_align(const int* ids, int* offsets, int* pos, int* sorted_tok,
-                               int n_pairs, int n_experts, int topk, hipStream_t stream) {
-  if (n_experts > ALIGN_MAX_EXPERTS) return -1;
+                               const float* weights, float* sorted_w, int n_pairs, int n_experts, int topk, hipStream_t stream) {
+  if (n_experts > ALIGN_MAX_EXPERTS || (sorted_w && !weights)) return -1;
   hipLaunchKernelGGL(moe_align_kernel, dim3(1), dim3(1024), 0, stream, ids, offsets, pos,
-                     sorted_tok, n_pairs, n_experts, topk);
+                     sorted_tok, weights, sorted_w, n_pairs, n_experts, topk);
   return 0;
 }
 
@@ -318,7 +321,8 @@ template <int TT>
 __global__ __launch_bounds__(256) void moe_mfma_gate_up_kernel(
     const uint16_t* __restrict__ x, const uint16_t* __restrict__ w13,
     const int* __restrict__ offsets, const int* __restrict__ sorted_tok,
-    uint16_t* __restrict__ act, int hidden, int inter, float act_limit, float act_alpha, float act_bias) {
+    uint16_t* __restrict__ act, int hidden, int inter, float act_limit, float act_alpha, float act_bias,
+    const float* __restrict__ row_scale) {
   const int e = blockIdx.y;
   const int r0 = offsets[e];
   const int n_e = offsets[e + 1] - r0;
@@ -366,9 +370,10 @@ __global__ __launch_bounds__(256) void moe_mfma_gate_up_kernel(
       const int j = t0 + tt * 16 + c16;
       if (tt < nt && j < n_e) {
         float v[4];
+        const float rs = row_scale ? row_scale[r0 + j] : 1.f;
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          float gt = accg[tt][r], up = accu[tt][r];
+          float gt = accg[tt][r] * rs, up = accu[tt][r] * rs;
           if (act_limit > 0.f) {  // clamped gated unit: min(g, limit) * sigmoid(alpha g) * (clamp(u) + bias)
             gt = fminf(gt, act_limit);
             up = fminf(fmaxf(up, -act_limit), act_limit) + act_bias;
@@ -449,10 +454,11 @@ __global__ __launch_bounds__(256) void moe_mfma_down_kernel(
 template <int TT>
 static void launch_moe_mfma(const void* x, const void* w13, const void* w2, const int* offsets,
                             const int* sorted_tok, void* act, void* y, int n_experts, int hidden,
-                            int inter, float act_limit, float act_alpha, float act_bias, hipStream_t stream) {
+                            int inter, float act_limit, float act_alpha, float act_bias, const float* row_scale,
+                            hipStream_t stream) {
   hipLaunchKernelGGL(moe_mfma_gate_up_kernel<TT>, dim3(inter / 64, n_experts), dim3(256), 0, stream,
                      (const uint16_t*)x, (const uint16_t*)w13, offsets, sorted_tok, (uint16_t*)act,
-                     hidden, inter, act_limit, act_alpha, act_bias);
+                     hidden, inter, act_limit, act_alpha, act_bias, row_scale);
   hipLaunchKernelGGL(moe_mfma_down_kernel<TT>, dim3(hidden / 16, n_experts), dim3(256), 0, stream,
                      (const uint16_t*)act, (const uint16_t*)w2, offsets, (uint16_t*)y, hidden, inter);
 }
@@ -460,11 +466,12 @@ static void launch_moe_mfma(const void* x, const void* w13, const void* w2, cons
 // x [tokens, hidden]; w13 [E, 2*inter, hidden]; w2 [E, hidden, inter]; offsets [E+1] and
 // sorted_tok [tokens*topk] from vpsa_moe_align; act [tokens*topk, inter] and
 // y [tokens*topk, hidden] are workspaces in expert-sorted row order.
-// act_limit > 0: the clamped gated unit (limit, alpha, bias) instead of SwiGLU.
+// act_limit > 0: the clamped gated unit (limit, alpha, bias) instead of SwiGLU.  row_scale (sorted order, or null):
+// gate and up of a row are multiplied by it before the activation (a factor on the row's input).
 VPSA_EXPORT int vpsa_moe_mfma_act(const void* x, const void* w13, const void* w2, const int* offsets,
                                   const int* sorted_tok, void* act, void* y, int tokens, int topk,
                                   int n_experts, int hidden, int inter, float act_limit, float act_alpha,
-                                  float act_bias, hipStream_t stream) {
+                                  float act_bias, const float* row_scale, hipStream_t stream) {
   if (tokens * topk <= 0) return 0;
   if (n_experts > ALIGN_MAX_EXPERTS) return -1;
   if (hidden % (32 * MOE_KU) != 0 || hidden % 16 != 0 || inter % 64 != 0 ||
@@ -473,13 +480,13 @@ VPSA_EXPORT int vpsa_moe_mfma_act(const void* x, const void* w13, const void* w2
   // an expert sees each token at most once: tokens bounds its row count
   if (tokens <= 16)
     launch_moe_mfma<1>(x, w13, w2, offsets, sorted_tok, act, y, n_experts, hidden, inter, act_limit, act_alpha,
-                       act_bias, stream);
+                       act_bias, row_scale, stream);
   else if (tokens <= 32)
     launch_moe_mfma<2>(x, w13, w2, offsets, sorted_tok, act, y, n_experts, hidden, inter, act_limit, act_alpha,
-                       act_bias, stream);
+                       act_bias, row_scale, stream);
   else
     launch_moe_mfma<4>(x, w13, w2, offsets, sorted_tok, act, y, n_experts, hidden, inter, act_limit, act_alpha,
-                       act_bias, stream);
+                       act_bias, row_scale, stream);
   return 0;
 }
 
@@ -488,5 +495,5 @@ VPSA_EXPORT int vpsa_moe_mfma(const void* x, const void* w13, const void* w2, co
                               int n_experts, int hidden, int inter, hipStream_t stream) {
   if (n_experts > MAX_EXPERTS) return -1;
   return vpsa_moe_mfma_act(x, w13, w2, offsets, sorted_tok, act, y, tokens, topk, n_experts, hidden, inter, 0.f,
-                           1.f, 0.f, stream);
+                           1.f, 0.f, nullptr, stream);
 }

@@ -34,6 +34,8 @@
 //   head_finish        head_rms with its parts optional: stabilised division by the normaliser column, unit RMS,
 //                      a weight per channel or per head and channel, a silu or sigmoid gate (a workgroup per head
 //                      from a thousand channels on)
+//   mingru             per channel S <- (1 - z) S + z cand(u) with z = sigmoid(z' + b_z), u = u' + b_u; y = S silu(g);
+//                      the state in the sequence's slot, long chunks in pieces side by side
 //
 // Plain kernels: every size is taken (bounds below are checked by the entry points).
 #include "common.h"
@@ -1174,6 +1176,221 @@ __global__ __launch_bounds__(256) void xielu_kernel(const T* __restrict__ x, T* 
   }
 }
 
+// ---------------------------------------------------------------------------------
+// minGRU: a gated recurrence whose gates read the current token only, so it is linear in its state:
+//   z = sigmoid(pz + bz), u = px + bx, cand = u + 1/2 where u >= 0 else sigmoid(u)
+//   S <- (1 - z) S + z cand (per channel),  y = S * silu(pg)
+// A run of tokens is a pair (A, B), S_end = A S_start + B, and runs compose.  A workgroup takes 128 neighbouring
+// channels (two per lane) and up to 128 rows at a time, its eight waves 16 rows each: gates and composites of the
+// rows stay in registers, the waves' composites meet in LDS, and each wave then walks its rows from its own start.
+// Sequences longer than a few blocks are cut into pieces of at most 128 rows (phase 1: composites of the pieces and
+// the sequences' start states, phase 2: start of the piece from the earlier pieces' composites, then its rows).
+// ---------------------------------------------------------------------------------
+#define GRU_ROWS 16
+#define GRU_WAVES 8
+#define GRU_BLOCK (GRU_ROWS * GRU_WAVES)
+#define GRU_COLS 128
+
+template <bool VEC, typename T>
+__device__ __forceinline__ void gru_ld2(const T* p, int c, int n, float* v) {
+  if constexpr (VEC && sizeof(T) == 2) {
+    const uint32_t u = c < n ? *reinterpret_cast<const uint32_t*>(p + c) : 0u;
+    v[0] = bf16lo(u);
+    v[1] = bf16hi(u);
+  } else {
+    v[0] = c < n ? Cv<T>::ld(p + c) : 0.f;
+    v[1] = c + 1 < n ? Cv<T>::ld(p + c + 1) : 0.f;
+  }
+}
+template <bool VEC, typename T>
+__device__ __forceinline__ void gru_st2(T* p, int c, int n, float a, float b) {
+  if constexpr (VEC && sizeof(T) == 2) {
+    if (c < n) *reinterpret_cast<uint32_t*>(p + c) = pack_bf16x2(a, b);
+  } else {
+    if (c < n) Cv<T>::st(p + c, a);
+    if (c + 1 < n) Cv<T>::st(p + c + 1, b);
+  }
+}
+__device__ __forceinline__ void gru_gates(float pz, float px, float& a, float& b) {
+  const float z = sigm(pz);
+  a = 1.f - z;
+  b = z * (px >= 0.f ? px + 0.5f : sigm(px));
+}
+
+// PHASE 0: blockIdx.x is a sequence, walked block by block; 1 / 2: blockIdx.x is a piece
+template <typename T, bool VEC, int PHASE>
+__global__ __launch_bounds__(512) void mingru_kernel(
+    const T* __restrict__ pz, const T* __restrict__ px, const T* __restrict__ pg, long stride, int width,
+    const float* __restrict__ bz, const float* __restrict__ bx, float* __restrict__ state, long state_stride,
+    const int* __restrict__ seq_cu, const int* __restrict__ seq_state, const int* __restrict__ positions,
+    T* __restrict__ y, const int* __restrict__ pieces, const int* __restrict__ seq_pieces, float* __restrict__ ws_a,
+    float* __restrict__ ws_b, float* __restrict__ ws_start) {
+  __shared__ float la[GRU_WAVES][GRU_COLS], lb[GRU_WAVES][GRU_COLS];
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+  const int c = blockIdx.y * GRU_COLS + 2 * lane;
+  const int bid = blockIdx.x;
+  int seq, row0, rows;
+  if (PHASE == 0) {
+    seq = bid;
+    row0 = seq_cu[seq];
+    rows = seq_cu[seq + 1] - row0;
+  } else {
+    seq = pieces[3 * bid];
+    row0 = pieces[3 * bid + 1];
+    rows = pieces[3 * bid + 2];
+  }
+  if (rows <= 0) return;
+  const int slot = seq_state[seq];
+  const bool fresh = slot < 0 || positions[seq_cu[seq]] == 0;
+  float* const st = state + (long)(slot < 0 ? 0 : slot) * state_stride;
+  const bool on[2] = {c < width, c + 1 < width};
+  float vz[2], vx[2], s[2] = {0.f, 0.f};
+#pragma unroll
+  for (int e = 0; e < 2; ++e) {
+    vz[e] = on[e] ? bz[c + e] : 0.f;
+    vx[e] = on[e] ? bx[c + e] : 0.f;
+  }
+  if (PHASE == 0 && !fresh) {
+#pragma unroll
+    for (int e = 0; e < 2; ++e) s[e] = on[e] ? st[c + e] : 0.f;
+  }
+  if (PHASE == 1 && bid == seq_pieces[seq] && wave == 0) {  // the slot is overwritten in phase 2: keep its value
+#pragma unroll
+    for (int e = 0; e < 2; ++e)
+      if (on[e]) ws_start[(long)seq * width + c + e] = fresh ? 0.f : st[c + e];
+  }
+  if (PHASE == 2) {
+#pragma unroll
+    for (int e = 0; e < 2; ++e) s[e] = on[e] ? ws_start[(long)seq * width + c + e] : 0.f;
+    const int p0 = seq_pieces[seq], n = bid - p0;
+    if (n > 0) {
+      const int q0 = p0 + n * wave / GRU_WAVES, q1 = p0 + n * (wave + 1) / GRU_WAVES;
+      float a[2] = {1.f, 1.f}, b[2] = {0.f, 0.f};
+      for (int q = q0; q < q1; ++q) {
+#pragma unroll
+        for (int e = 0; e < 2; ++e)
+          if (on[e]) {
+            const float pa = ws_a[(long)q * width + c + e];
+            b[e] = pa * b[e] + ws_b[(long)q * width + c + e];
+            a[e] *= pa;
+          }
+      }
+#pragma unroll
+      for (int e = 0; e < 2; ++e) la[wave][2 * lane + e] = a[e], lb[wave][2 * lane + e] = b[e];
+      __syncthreads();
+#pragma unroll
+      for (int w = 0; w < GRU_WAVES; ++w)
+#pragma unroll
+        for (int e = 0; e < 2; ++e) s[e] = la[w][2 * lane + e] * s[e] + lb[w][2 * lane + e];
+      __syncthreads();
+    }
+  }
+  for (int r0 = 0; r0 < rows; r0 += GRU_BLOCK) {
+    const int w0 = r0 + GRU_ROWS * wave;
+    const int cnt = min(GRU_ROWS, rows - w0);  // rows of this wave (may be <= 0)
+    const long at = (long)(row0 + w0) * stride;
+    float a[GRU_ROWS][2], b[GRU_ROWS][2], g[GRU_ROWS][2];
+#pragma unroll
+    for (int i = 0; i < GRU_ROWS; ++i) {
+#pragma unroll
+      for (int e = 0; e < 2; ++e) a[i][e] = b[i][e] = g[i][e] = 0.f;
+      if (i < cnt) {
+        gru_ld2<VEC>(pz + at + i * stride, c, width, a[i]);
+        gru_ld2<VEC>(px + at + i * stride, c, width, b[i]);
+        if (PHASE != 1) gru_ld2<VEC>(pg + at + i * stride, c, width, g[i]);
+      }
+    }
+    float ca[2] = {1.f, 1.f}, cb[2] = {0.f, 0.f};
+#pragma unroll
+    for (int i = 0; i < GRU_ROWS; ++i)
+      if (i < cnt) {
+#pragma unroll
+        for (int e = 0; e < 2; ++e) {
+          gru_gates(a[i][e] + vz[e], b[i][e] + vx[e], a[i][e], b[i][e]);
+          cb[e] = a[i][e] * cb[e] + b[i][e];
+          ca[e] *= a[i][e];
+        }
+      }
+#pragma unroll
+    for (int e = 0; e < 2; ++e) la[wave][2 * lane + e] = ca[e], lb[wave][2 * lane + e] = cb[e];
+    __syncthreads();
+    if (PHASE == 1) {
+      if (wave == 0) {
+        float ta[2] = {1.f, 1.f}, tb[2] = {0.f, 0.f};
+#pragma unroll
+        for (int w = 0; w < GRU_WAVES; ++w)
+#pragma unroll
+          for (int e = 0; e < 2; ++e) {
+            const float wa = la[w][2 * lane + e];
+            tb[e] = wa * tb[e] + lb[w][2 * lane + e];
+            ta[e] *= wa;
+          }
+#pragma unroll
+        for (int e = 0; e < 2; ++e)
+          if (on[e]) ws_a[(long)bid * width + c + e] = ta[e], ws_b[(long)bid * width + c + e] = tb[e];
+      }
+      return;  // a piece is at most one block
+    }
+    float mine[2] = {s[0], s[1]};
+#pragma unroll
+    for (int w = 0; w < GRU_WAVES; ++w) {
+#pragma unroll
+      for (int e = 0; e < 2; ++e) {
+        s[e] = la[w][2 * lane + e] * s[e] + lb[w][2 * lane + e];
+        if (w + 1 == wave) mine[e] = s[e];
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < GRU_ROWS; ++i)
+      if (i < cnt) {
+        float o[2];
+#pragma unroll
+        for (int e = 0; e < 2; ++e) {
+          mine[e] = a[i][e] * mine[e] + b[i][e];
+          o[e] = mine[e] * g[i][e] * sigm(g[i][e]);
+        }
+        gru_st2<VEC>(y + (long)(row0 + w0 + i) * width, c, width, o[0], o[1]);
+      }
+    __syncthreads();  // the composites are rewritten by the next block
+  }
+  if (PHASE == 1) return;
+  if (wave == 0 && slot >= 0 && (PHASE == 0 || bid + 1 == seq_pieces[seq + 1])) {
+#pragma unroll
+    for (int e = 0; e < 2; ++e)
+      if (on[e]) st[c + e] = s[e];
+  }
+}
+
+// One row per sequence (row i is sequence i): a thread per two channels
+template <typename T, bool VEC>
+__global__ __launch_bounds__(256) void mingru_step_kernel(
+    const T* __restrict__ pz, const T* __restrict__ px, const T* __restrict__ pg, long stride, int width,
+    const float* __restrict__ bz, const float* __restrict__ bx, float* __restrict__ state, long state_stride,
+    const int* __restrict__ seq_state, const int* __restrict__ positions, T* __restrict__ y) {
+  const long row = blockIdx.y;
+  const int c = (blockIdx.x * 256 + threadIdx.x) * 2;
+  if (c >= width) return;
+  const int slot = seq_state[row];
+  const bool fresh = slot < 0 || positions[row] == 0;
+  float* const st = state + (long)(slot < 0 ? 0 : slot) * state_stride;
+  float z[2], x[2], g[2], o[2];
+  gru_ld2<VEC>(pz + row * stride, c, width, z);
+  gru_ld2<VEC>(px + row * stride, c, width, x);
+  gru_ld2<VEC>(pg + row * stride, c, width, g);
+#pragma unroll
+  for (int e = 0; e < 2; ++e) {
+    o[e] = 0.f;
+    if (c + e < width) {
+      float a, b;
+      gru_gates(z[e] + bz[c + e], x[e] + bx[c + e], a, b);
+      const float s = fresh ? b : a * st[c + e] + b;
+      if (slot >= 0) st[c + e] = s;
+      o[e] = s * g[e] * sigm(g[e]);
+    }
+  }
+  gru_st2<VEC>(y + row * width, c, width, o[0], o[1]);
+}
+
 }  // namespace
 
 #define SM_DISPATCH(dt, CALL)                         \
@@ -1512,5 +1729,44 @@ VPSA_EXPORT int vpsa_xielu(const void* x, void* y, long n, const float* act, int
   long blocks = (n + 255) / 256;
   if (blocks > 65536) blocks = 65536;
   SM_DISPATCH(dt, (xielu_kernel<T><<<(unsigned)blocks, 256, 0, stream>>>((const T*)x, (T*)y, n, act)));
+  return 0;
+}
+
+// pz, px, pg: column ranges of one projection (row stride `stride`).  n_seqs == rows: every sequence has one row.
+// n_pieces > 0: pieces int32 [n_pieces, 3] = (sequence, first row, rows <= 128), in order and covering every sequence,
+// seq_pieces [n_seqs + 1] = a sequence's first piece; ws_a, ws_b [n_pieces, width], ws_start [n_seqs, width] scratch.
+VPSA_EXPORT int vpsa_mingru(const void* pz, const void* px, const void* pg, long stride, int width, const float* bz,
+                            const float* bx, float* state, long state_stride, const int* seq_cu, const int* seq_state,
+                            int n_seqs, const int* positions, void* y, int rows, const int* pieces,
+                            const int* seq_pieces, int n_pieces, float* ws_a, float* ws_b, float* ws_start, int dtype,
+                            hipStream_t st) {
+  if (rows <= 0 || n_seqs <= 0) return 0;
+  if (dtype != 0 && dtype != 1) return -2;
+  if (width <= 0 || n_seqs > rows || (n_pieces > 0 && (!pieces || !seq_pieces || !ws_a || !ws_b || !ws_start))) return -1;
+  const bool vec = width % 2 == 0 && stride % 2 == 0 &&
+                   (((uintptr_t)pz | (uintptr_t)px | (uintptr_t)pg | (uintptr_t)y) & 3) == 0;
+  const int cols = (width + GRU_COLS - 1) / GRU_COLS;
+#define GRU_PH(T, V, P, N)                                                                                       \
+  mingru_kernel<T, V, P><<<dim3(N, cols), 512, 0, st>>>((const T*)pz, (const T*)px, (const T*)pg, stride, width, \
+                                                        bz, bx, state, state_stride, seq_cu, seq_state,          \
+                                                        positions, (T*)y, pieces, seq_pieces, ws_a, ws_b, ws_start)
+#define GRU_GO(T, V)                                                                                                 \
+  do {                                                                                                               \
+    if (n_seqs == rows && rows <= 65535) {                                                                           \
+      mingru_step_kernel<T, V><<<dim3((width + 511) / 512, rows), 256, 0, st>>>(                                     \
+          (const T*)pz, (const T*)px, (const T*)pg, stride, width, bz, bx, state, state_stride, seq_state,           \
+          positions, (T*)y);                                                                                         \
+    } else if (n_pieces > 0) {                                                                                       \
+      GRU_PH(T, V, 1, n_pieces);                                                                                     \
+      GRU_PH(T, V, 2, n_pieces);                                                                                     \
+    } else {                                                                                                         \
+      GRU_PH(T, V, 0, n_seqs);                                                                                       \
+    }                                                                                                                \
+  } while (0)
+  if (dtype == 1) GRU_GO(float, false);
+  else if (vec) GRU_GO(bf16_t, true);
+  else GRU_GO(bf16_t, false);
+#undef GRU_GO
+#undef GRU_PH
   return 0;
 }

@@ -65,7 +65,8 @@ __global__ __launch_bounds__(512, 2) void tile_gemm_kernel(
     const uint16_t* __restrict__ a, long lda, const int* __restrict__ arow_idx,
     const uint16_t* __restrict__ w, long w_group_stride, const int* __restrict__ offsets, int n_groups, int max_rows,
     uint16_t* __restrict__ c, long ldc, const uint16_t* __restrict__ resid, long ldr,
-    int n_total, int k_total, int n_tiles, float act_limit, float act_alpha, float act_bias) {
+    int n_total, int k_total, int n_tiles, float act_limit, float act_alpha, float act_bias,
+    const float* __restrict__ row_scale) {
   extern __shared__ __attribute__((aligned(1024))) char lds[];
   const int tid = threadIdx.x;
   const int lane = tid & 63;
@@ -300,14 +301,15 @@ __global__ __launch_bounds__(512, 2) void tile_gemm_kernel(
       if (TG_PAIRED(EPI)) {
         const int col = n_idx * 128 + wc * 32 + 8 * fq;
         float v[8];
+        const float rs = (EPI == TG_EPI_GLU_CLAMP && row_scale && row < row_end) ? row_scale[row] : 1.f;
 #pragma unroll
         for (int ni = 0; ni < 2; ++ni)
 #pragma unroll
           for (int e = 0; e < 4; ++e) {
             float gt = acc[mh][0][mi][ni][e], up = acc[mh][1][mi][ni][e];
             if (EPI == TG_EPI_GLU_CLAMP) {
-              gt = fminf(gt, act_limit);
-              up = fminf(fmaxf(up, -act_limit), act_limit) + act_bias;
+              gt = fminf(gt * rs, act_limit);
+              up = fminf(fmaxf(up * rs, -act_limit), act_limit) + act_bias;
               v[4 * ni + e] = gt / (1.f + __expf(-act_alpha * gt)) * up;
             } else if (EPI == TG_EPI_GELU_GLU) {
               // 0.5 g (1 + tanh(y)) = g / (1 + exp(-2 y)),  y = sqrt(2 / pi) (g + 0.044715 g^3)
@@ -374,17 +376,19 @@ VPSA_EXPORT int vpsa_tile_gemm_debug(int v) {
 // offsets[G] <= max_rows, or null (one group of max_rows rows); c [max_rows, N] (SwiGLU: N / 2
 // columns), row stride ldc; epi: 0 store, 1 SwiGLU, 2 store of product + resid (row stride ldr; may
 // alias c), 6 gated gelu unit (tanh form, paired like SwiGLU), 3 clamped gated unit (paired like SwiGLU, constants act_*), 4 squared ReLU, 5 xIELU (act_alpha, act_bias: its two curvatures).  Every byte offset into a and into one group of w must fit 32 bits.
+// row_scale fp32 [max_rows] or null (epi 3 only): gate and up of output row r are multiplied by row_scale[r] before the
+// clamps, i.e. the row's input carries that factor.
 // Returns 0, or a negative number when the shape is outside what the kernel tiles.
 VPSA_EXPORT int vpsa_tile_gemm(const void* a, long lda, const void* arow_idx, const void* w, const void* offsets,
                                int n_groups, void* c, long ldc, int max_rows, int n, int k, int epi, const void* resid,
                                long ldr, long a_rows, float act_limit, float act_alpha, float act_bias,
-                               hipStream_t stream) {
+                               const void* row_scale, hipStream_t stream) {
   if (k % TG_BK != 0 || k <= 0 || n <= 0 || max_rows <= 0 || n_groups <= 0 || lda % 8 != 0 || ldc % 8 != 0) return -1;
   if (!offsets && n_groups != 1) return -1;
   if (TG_PAIRED(epi) && (n % 2 != 0 || (n / 2) % 32 != 0)) return -1;
   if (!TG_PAIRED(epi) && n % 8 != 0) return -1;
   if (epi == TG_EPI_RESIDUAL && (!resid || ldr % 8 != 0)) return -1;
-  if (epi < 0 || epi > 6) return -1;
+  if (epi < 0 || epi > 6 || (row_scale && epi != TG_EPI_GLU_CLAMP)) return -1;
   if ((double)a_rows * (double)lda * 2.0 >= 4294967296.0 || (double)n * (double)k * 2.0 >= 4294967296.0) return -1;
   const int n_tiles = TG_PAIRED(epi) ? (n / 2 + 127) / 128 : (n + TG_BN - 1) / TG_BN;
   const int m_tiles_max = offsets ? max_rows / TG_BM + n_groups : (max_rows + TG_BM - 1) / TG_BM;
@@ -402,7 +406,8 @@ VPSA_EXPORT int vpsa_tile_gemm(const void* a, long lda, const void* arow_idx, co
     }                                                                                                                \
     tile_gemm_kernel<E, D><<<dim3((unsigned)blocks), dim3(512), TG_LDS, stream>>>(                                       \
         (const uint16_t*)a, lda, (const int*)arow_idx, (const uint16_t*)w, wstride, (const int*)offsets, n_groups,   \
-        max_rows, (uint16_t*)c, ldc, (const uint16_t*)resid, ldr, n, k, n_tiles, act_limit, act_alpha, act_bias);    \
+        max_rows, (uint16_t*)c, ldc, (const uint16_t*)resid, ldr, n, k, n_tiles, act_limit, act_alpha, act_bias,    \
+        (const float*)row_scale);                                                                                    \
   } while (0)
   if (epi == TG_EPI_SWIGLU) TG_LAUNCH(TG_EPI_SWIGLU, 0);
   else if (epi == TG_EPI_RESIDUAL) TG_LAUNCH(TG_EPI_RESIDUAL, 0);

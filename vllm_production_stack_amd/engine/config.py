@@ -18,8 +18,8 @@ import torch
 
 @dataclass(frozen=True)
 class LatentMixerSpec:
-    """A latent-attention mixer: queries and keys/values pass through low-rank latents; a head's
-    query/key has ``dim`` unrotated and ``rot_dim`` rotated channels (the rotated key part is one
+    """A latent-attention mixer: queries (unless ``q_rank`` is 0: one projection) and keys/values pass through
+    low-rank latents; a head's query/key has ``dim`` unrotated and ``rot_dim`` rotated channels (the rotated key part is one
     vector shared by all heads), its value ``vdim`` channels.  Only the KV latent (``kv_rank``) and
     the rotated key part are cached.  ``kv_from``: the layer whose cache entries this layer reads
     instead of writing its own (it then has no KV down-projection)."""
@@ -35,15 +35,33 @@ class LatentMixerSpec:
     kv_from: int | None = None
     sink: bool = True          # a learned per-head logit in the softmax denominator
     out_gate: bool = True      # head outputs times sigmoid(W_g h)
+    rope_layout: str = "pairs"  # checkpoint order of the rotated channels: "pairs" (2 i, 2 i + 1) or "half" (i, i + dims / 2)
 
     @property
     def entry(self) -> int:    # cached values per token
         return self.kv_rank + self.rot_dim
 
     def weight_count(self, width: int) -> int:
-        n = width * (self.q_rank + self.heads) + self.q_rank * self.heads * (self.dim + self.rot_dim)
+        q_in = self.q_rank if self.q_rank else width   # what the head queries are projected from
+        n = width * (self.q_rank + (self.heads if self.out_gate else 0)) + q_in * self.heads * (self.dim + self.rot_dim)
         n += self.heads * self.vdim * width + self.heads * self.kv_rank * (self.dim + self.vdim)
         return n + (width * self.entry if self.kv_from is None else 0)
+
+
+@dataclass(frozen=True)
+class MinGRUSpec:
+    """A gated recurrence over ``width`` channels whose gates read the current token only: z = sigmoid(W_z h + b_z),
+    candidate from u = W_x h + b_x, S <- (1 - z) S + z candidate; the output is projected from S silu(W_g h)."""
+    width: int
+
+    def state_elems(self) -> int:
+        return self.width
+
+    def weight_count(self, width: int) -> int:
+        return 4 * width * self.width
+
+    def token_flops(self) -> float:
+        return 4.0 * self.width
 
 
 @dataclass(frozen=True)
@@ -53,7 +71,8 @@ class FeedForwardSpec:
     an always-on shared unit of width ``shared_ff`` (0 = none) with a per-token sigmoid gate."""
     kind: str = "dense"
     ff: int = 0
-    act: str = "relu_sq"       # relu_sq | xielu (two learned curvatures, see ops.xielu) | gelu_tanh | silu (gated units)
+    act: str = "relu_sq"       # relu_sq | xielu (two learned curvatures, see ops.xielu) | poly_norm (four learned
+                               # numbers, see ops.poly_norm) | gelu_tanh | silu (gated units)
     gated: bool = False        # down(act(gate x) * (up x)) instead of down(act(up x))
     router: str = "sigmoid"    # sigmoid: as described above | softmax: softmax scores, a learned selection bias,
                                # a group scores its largest biased score, weights = scores, not renormalised
@@ -64,6 +83,7 @@ class FeedForwardSpec:
     keep: int = 1
     route_scale: float = 1.0
     norm_topk: bool = False    # sigmoid router: the chosen scores are divided by their sum (+ 1e-20) first
+    scale_input: bool = False  # a routing weight multiplies its unit's input instead of its output
     limit: float = 0.0
     shared_ff: int = 0
     shared_limit: float = 0.0
@@ -463,6 +483,59 @@ def zetalorn_config(name: str, vocab: int, width: int, layers: list[dict], loop:
         bos_token_id=0, eos_token_id=-1)  # the design names no special tokens
 
 
+def zupilorn_layers(layers: list[dict]) -> tuple:
+    """The ``layers`` list of a Zupilorn config.json -> layer specs."""
+    out = []
+    for i, entry in enumerate(layers):
+        m = entry["mixer"]
+        kind = entry["type"]
+        if kind == "latent_attention":
+            rot = m["rot"]
+            mixer = LatentMixerSpec(
+                heads=int(m["heads"]), dim=int(m["dim"]), rot_dim=int(m["rot_dim"]), vdim=int(m["vdim"]),
+                kv_rank=int(m["kv_rank"]), q_rank=0, rope_base=float(rot["base"]),
+                rope_dims=int(rot.get("dims", m["rot_dim"])), scale=float(m["scale"]), sink=False, out_gate=False,
+                rope_layout="half")
+            _positive(i, heads=mixer.heads, dim=mixer.dim, rot_dim=mixer.rot_dim, vdim=mixer.vdim, kv_rank=mixer.kv_rank)
+            if mixer.rope_dims % 2 or not 0 < mixer.rope_dims <= mixer.rot_dim:
+                raise ValueError(f"layer {i}: rotary dims must be even and within rot_dim")
+        elif kind == "mingru":
+            mixer = MinGRUSpec(int(m["width"]))
+            _positive(i, width=mixer.width)
+        else:
+            raise ValueError(f"layer {i}: unknown mixer type {kind!r}")
+        f = entry.get("mlp")
+        mlp = None
+        if f is not None:
+            if f["kind"] == "dense":
+                mlp = FeedForwardSpec(kind="dense", ff=int(f["ff"]), act="poly_norm")
+            elif f["kind"] == "moe":
+                r, ex = f["router"], f["expert"]
+                mlp = FeedForwardSpec(kind="moe", ff=int(ex["ff"]), gated=True, experts=int(r["experts"]), top=int(r["top"]),
+                                      scale_input=True, limit=float(ex["limit"]))
+                if not 1 <= mlp.top <= mlp.experts or mlp.limit <= 0:
+                    raise ValueError(f"layer {i}: 1 <= top <= experts and a positive limit are required")
+            else:
+                raise ValueError(f"layer {i}: unknown feed-forward kind {f['kind']!r}")
+            _positive(i, ff=mlp.ff)
+        out.append(LayerSpec(kind, mixer, mlp))
+    return tuple(out)
+
+
+def zupilorn_config(name: str, vocab: int, width: int, layers: list[dict], logit_softcap: float | None = None,
+                    norm_eps: float = 1e-5, max_position_embeddings: int = 32768) -> "ModelConfig":
+    specs = zupilorn_layers(layers)
+    att = [s.mixer for s in specs if isinstance(s.mixer, LatentMixerSpec)]
+    return ModelConfig(
+        name=name, architecture="zupilorn", vocab_size=int(vocab), hidden_size=int(width),
+        intermediate_size=max([s.mlp.ff for s in specs if s.mlp] + [0]), num_layers=len(specs),
+        num_heads=max([m.heads for m in att] + [1]), num_kv_heads=1,
+        head_dim=max([m.dim + m.rot_dim for m in att] + [64]), norm_eps=float(norm_eps),
+        max_position_embeddings=max_position_embeddings, tie_word_embeddings=True,
+        logit_softcap=float(logit_softcap or 0.0), layer_specs=specs,
+        bos_token_id=0, eos_token_id=-1)  # the design names no special tokens
+
+
 def _rotary(rot: dict, layout: str) -> RotarySpec:
     sc = rot.get("scaling")
     scaling = None if not sc else (float(sc["factor"]), float(sc["original"]), float(sc["fast"]), float(sc["slow"]))
@@ -574,7 +647,7 @@ def zururax_config(name: str, vocab: int, width: int, layers: list[dict], embedd
 @dataclass
 class ModelConfig:
     name: str = "tiny-llama"
-    architecture: str = "llama"  # llama | mixtral | opt | gpt2 | zururax | revelix | pelatar | zetalorn
+    architecture: str = "llama"  # llama | mixtral | opt | gpt2 | zururax | revelix | pelatar | zetalorn | zupilorn
     vocab_size: int = 512
     hidden_size: int = 256
     intermediate_size: int = 512
@@ -601,6 +674,7 @@ class ModelConfig:
     layer_specs: tuple = ()
     embedding_scale: float = 1.0
     logit_scale: float = 1.0   # logits = head(x) * logit_scale
+    logit_softcap: float = 0.0  # logits <- cap tanh(logits / cap), 0 = none
     # (start, stop, times): layers start .. stop - 1 run `times` times in a row with the same weights, every pass
     # with cache entries and state of its own
     layer_loop: tuple | None = None
@@ -903,6 +977,36 @@ PRESETS["tiny-zetalorn"] = zetalorn_config(
 PRESETS["zetalorn-bench"] = zetalorn_config("zetalorn-bench", 32000, 2048, zetalorn_stack(2048, 16, 16, 1024, 4),
                                             loop={"start": 0, "stop": 2, "times": 2}, logit_scale=0.5)
 
+
+def _zp_attention(heads, dim, rot_dim, vdim, kv_rank, mlp=None, base=10000.0):
+    return {"type": "latent_attention", "mlp": mlp,
+            "mixer": {"heads": heads, "dim": dim, "rot_dim": rot_dim, "vdim": vdim, "kv_rank": kv_rank,
+                      "rot": {"base": base, "dims": rot_dim}, "scale": (dim + rot_dim) ** -0.5}}
+
+
+def _zp_moe(ff, experts, top, limit=7.0):
+    return {"kind": "moe", "expert": {"ff": ff, "limit": limit}, "router": {"experts": experts, "top": top}}
+
+
+def zupilorn_stack(width, heads, ff, experts, unit_ff, top, blocks=1):
+    """Layer list of a Zupilorn at random weights: per block a latent attention layer with a dense feed-forward and a
+    minGRU layer, as wide as the model, with routed units."""
+    out = []
+    for _ in range(blocks):
+        out += [_zp_attention(heads, 128, 64, 128, 512, {"kind": "dense", "ff": ff}),
+                {"type": "mingru", "mixer": {"width": width}, "mlp": _zp_moe(unit_ff, experts, top)}]
+    return out
+
+
+# Zupilorn at random weights: a small one for smoke runs, and one with layer shapes of a 2048-wide model
+PRESETS["tiny-zupilorn"] = zupilorn_config(
+    "tiny-zupilorn", 512, 192,
+    [{"type": "mingru", "mixer": {"width": 160}, "mlp": _zp_moe(64, 6, 2, 2.0)},
+     _zp_attention(3, 24, 32, 40, 64, {"kind": "dense", "ff": 384}),
+     {"type": "mingru", "mixer": {"width": 64}, "mlp": None}], logit_softcap=20.0, max_position_embeddings=4096)
+PRESETS["zupilorn-bench"] = zupilorn_config("zupilorn-bench", 32000, 2048, zupilorn_stack(2048, 16, 5120, 16, 1024, 4, 2),
+                                            logit_softcap=30.0)
+
 _ALIASES = {
     "meta-llama/meta-llama-3-8b": "llama-3-8b",
     "meta-llama/meta-llama-3-8b-instruct": "llama-3-8b",
@@ -940,6 +1044,10 @@ def _from_hf_config(cfg: dict[str, Any], name: str) -> ModelConfig:
     if str(cfg.get("architecture", "")).lower() == "zetalorn":
         return zetalorn_config(name, cfg["vocab"], cfg["width"], cfg["layers"], loop=cfg.get("loop"),
                                logit_scale=cfg.get("logit_scale", 1.0), norm_eps=(cfg.get("norm") or {}).get("eps", 1e-6),
+                               max_position_embeddings=int(cfg.get("max_positions", 32768)))
+    if str(cfg.get("architecture", "")).lower() == "zupilorn":
+        return zupilorn_config(name, cfg["vocab"], cfg["width"], cfg["layers"], logit_softcap=cfg.get("logit_softcap"),
+                               norm_eps=(cfg.get("norm") or {}).get("eps", 1e-5),
                                max_position_embeddings=int(cfg.get("max_positions", 32768)))
     if str(cfg.get("architecture", "")).lower() == "pelatar":
         return pelatar_config(name, cfg["vocab"], cfg["width"], cfg["layers"],

@@ -20,6 +20,7 @@ from .transformer import LayerWeights, TransformerModel
 from .pelatar import PelatarModel
 from .revelix import RevelixModel
 from .zetalorn import ZetalornModel
+from .zupilorn import ZupilornModel
 from .zururax import ZururaxModel
 
 
@@ -36,6 +37,8 @@ def build_model(cfg: ModelConfig, dtype: torch.dtype, device: torch.device, max_
         model = PelatarModel(cfg, dtype, device, max_model_len)
     elif cfg.architecture == "zetalorn":
         model = ZetalornModel(cfg, dtype, device, max_model_len)
+    elif cfg.architecture == "zupilorn":
+        model = ZupilornModel(cfg, dtype, device, max_model_len)
     else:
         model = TransformerModel(cfg, dtype, device, max_model_len, expert_parallel=expert_parallel)
     has_weights = ckpt_dir is not None and any(Path(ckpt_dir).glob("*.safetensors"))
@@ -73,6 +76,8 @@ def load_hf_weights(model, ckpt_dir: Path) -> None:
         _load_pelatar(model, ckpt_dir)
     elif isinstance(model, ZetalornModel):
         _load_zetalorn(model, ckpt_dir)
+    elif isinstance(model, ZupilornModel):
+        _load_zupilorn(model, ckpt_dir)
     else:
         _load_llama(model, ckpt_dir)
 
@@ -238,6 +243,11 @@ def _load_gpt2(model: OPTModel, ckpt_dir: Path) -> None:
                 model.layers[int(m.group(1))][key].copy_(t.t() if transpose else t)
 
 
+def heads_transposed(t: torch.Tensor, heads: int) -> torch.Tensor:
+    """A per-head projection [heads * out, in] as [heads, in, out], the right operand of a batched product."""
+    return t.view(heads, -1, t.shape[1]).transpose(1, 2)
+
+
 def _load_zururax(model: ZururaxModel, ckpt_dir: Path) -> None:
     """Zururax checkpoints: ``embed``, ``l<i>.norm1|norm2``, ``l<i>.mix.{dq, dq.norm, uq, dkv, dkv.norm, uk, uv,
     sink, g, o}``, ``l<i>.mlp.{up, down}`` or ``l<i>.mlp.{router, e<k>.{gate, up, down}, shared.{gate, up, down,
@@ -288,7 +298,7 @@ def _load_zururax(model: ZururaxModel, ckpt_dir: Path) -> None:
             elif sub == "mix.uk":
                 put(lw.w_uk.view(m.heads * m.dim, m.kv_rank), t, name)
             elif sub == "mix.uv":
-                put(lw.w_uv.view(m.heads * m.vdim, m.kv_rank), t, name)
+                put(lw.w_uv, heads_transposed(t, m.heads), name)
             elif sub == "mix.sink" and m.sink:
                 put(lw.sink, t, name)
             elif sub == "mix.o":
@@ -711,3 +721,92 @@ def _load_zetalorn(model: ZetalornModel, ckpt_dir: Path) -> None:
             want |= {f"l{i}.mlp.e{e}.{k}" for e in range(f.experts) for k in ("gate", "up", "down")}
     if want - seen:
         raise ValueError(f"checkpoint lacks {sorted(want - seen)[:8]}")
+
+
+def half_to_pairs(t: torch.Tensor, dims: int) -> torch.Tensor:
+    """Rows [..., n, in] of a projection whose first ``dims`` channels rotate in pairs (i, i + dims / 2), reordered so
+    that partners are neighbours, (2 i, 2 i + 1).  Query and key rows reordered alike give the same products."""
+    order = torch.arange(dims).view(2, -1).t().reshape(-1)
+    order = torch.cat([order, torch.arange(dims, t.shape[-2])])
+    return t.index_select(-2, order)
+
+
+def _load_zupilorn(model: ZupilornModel, ckpt_dir: Path) -> None:
+    """Zupilorn checkpoints: ``embed``, ``embed.norm``, ``final.norm``; per layer ``l<i>.norm1|norm1b`` (and, with a
+    feed-forward, ``norm2|norm2b``), ``l<i>.dwa`` (depth average), ``l<i>.mix.{q, dkv, dkv.norm, uk, uv, o}`` (latent
+    attention) or ``l<i>.mix.{z, z.b, x, x.b, g, o}`` (minGRU), ``l<i>.mlp.{up, down, act}`` or ``l<i>.mlp.router`` and
+    ``l<i>.mlp.e<j>.{gate, up, down}``.  Linear weights are [out, in]; a mixer's input projections are fused row-wise
+    here and the units stacked.  The model's norms are stored around zero (gain 1 + w), the latent's as it is.
+    Every tensor the model holds must be found, and every tensor of the file must have a place."""
+    from ..engine.config import MinGRUSpec
+
+    def put(dst: torch.Tensor, src: torch.Tensor, what: str) -> None:
+        if tuple(dst.shape) != tuple(src.shape):
+            raise ValueError(f"{what}: checkpoint shape {tuple(src.shape)}, model expects {tuple(dst.shape)}")
+        dst.copy_(src.to(dst.dtype))
+
+    def put_gain(dst: torch.Tensor, src: torch.Tensor, what: str) -> None:
+        put(dst, 1.0 + src.float(), what)
+
+    places: dict = {"embed": lambda t, n: put(model.embed, t, n),
+                    "embed.norm": lambda t, n: put_gain(model.embed_norm, t, n),
+                    "final.norm": lambda t, n: put_gain(model.norm, t, n)}
+
+    def layer_places(lw) -> dict:
+        m, f = lw.spec.mixer, lw.spec.mlp
+        out = {"norm1": (put_gain, lw.norm1), "norm1b": (put_gain, lw.norm1b), "dwa": (put, lw.dwa), "mix.o": (put, lw.w_o)}
+        if isinstance(m, MinGRUSpec):
+            for k, name in enumerate(("z", "x", "g")):
+                out[f"mix.{name}"] = (put, lw.w_in[k * m.width:(k + 1) * m.width])
+            out["mix.z.b"], out["mix.x.b"] = (put, lw.z_bias), (put, lw.x_bias)
+        else:
+            nq = m.heads * (m.dim + m.rot_dim)
+
+            def put_q(dst, t, n):
+                if tuple(t.shape) != tuple(dst.shape):
+                    raise ValueError(f"{n}: checkpoint shape {tuple(t.shape)}, model expects {tuple(dst.shape)}")
+                if m.rope_layout == "half":
+                    t = t.view(m.heads, m.dim + m.rot_dim, -1)
+                    t = torch.cat([t[:, :m.dim], half_to_pairs(t[:, m.dim:], m.rope_dims)], dim=1).reshape(nq, -1)
+                put(dst, t, n)
+
+            def put_dkv(dst, t, n):
+                if tuple(t.shape) != tuple(dst.shape):
+                    raise ValueError(f"{n}: checkpoint shape {tuple(t.shape)}, model expects {tuple(dst.shape)}")
+                if m.rope_layout == "half":
+                    t = torch.cat([t[:m.kv_rank], half_to_pairs(t[m.kv_rank:], m.rope_dims)])
+                put(dst, t, n)
+
+            def put_uv(dst, t, n):
+                if tuple(t.shape) != (m.heads * m.vdim, m.kv_rank):
+                    raise ValueError(f"{n}: checkpoint shape {tuple(t.shape)}, model expects {(m.heads * m.vdim, m.kv_rank)}")
+                put(dst, heads_transposed(t, m.heads), n)
+
+            out["mix.q"] = (put_q, lw.w_in[:nq])
+            out["mix.dkv"] = (put_dkv, lw.w_in[nq:nq + m.entry])
+            out["mix.dkv.norm"] = (put, lw.dkv_norm)
+            out["mix.uk"] = (put, lw.w_uk.view(m.heads * m.dim, m.kv_rank))
+            out["mix.uv"] = (put_uv, lw.w_uv)
+        if f is not None:
+            out["norm2"], out["norm2b"] = (put_gain, lw.norm2), (put_gain, lw.norm2b)
+            if f.kind == "dense":
+                out["mlp.up"], out["mlp.down"], out["mlp.act"] = (put, lw.w_up), (put, lw.w_down), (put, lw.act)
+            else:
+                out["mlp.router"] = (put, lw.router)
+                for e in range(f.experts):
+                    out[f"mlp.e{e}.gate"] = (put, lw.w13[e, :f.ff])
+                    out[f"mlp.e{e}.up"] = (put, lw.w13[e, f.ff:])
+                    out[f"mlp.e{e}.down"] = (put, lw.w2[e])
+        return out
+
+    for i, lw in enumerate(model.layers):
+        for sub, (how, dst) in layer_places(lw).items():
+            places[f"l{i}.{sub}"] = lambda t, n, how=how, dst=dst: how(dst, t, n)
+    seen = set()
+    for name, t in _iter_safetensors(ckpt_dir):
+        if name not in places:
+            raise ValueError(f"unexpected tensor {name!r}")
+        places[name](t, name)
+        seen.add(name)
+    if set(places) - seen:
+        raise ValueError(f"checkpoint lacks {sorted(set(places) - seen)[:8]}")

@@ -44,6 +44,7 @@ def _kernels():
             "vpsa_add_dyt", "vpsa_recurrent_scan", "vpsa_head_rms", "vpsa_short_conv_qkv", "vpsa_window_attention",
             "vpsa_mix_heads", "vpsa_xielu", "vpsa_window_mfma_supported", "vpsa_window_attention_mfma", "vpsa_window_tile_slots",
             "vpsa_gated_add_rmsnorm", "vpsa_pool_blocks", "vpsa_diff_heads",
+            "vpsa_embed_rmsnorm", "vpsa_depth_mix_rmsnorm", "vpsa_poly_norm", "vpsa_soft_cap", "vpsa_mingru",
         ):
             getattr(lib, name).restype = c_int
         lib.vpsa_prefill_split_record_bytes.restype = c_long
@@ -1067,8 +1068,9 @@ def moe_localize(ids, weights, first, count, bucket):
             torch.where(here, weights, 0.0).to(weights.dtype))
 
 
-def moe_align(ids, n_experts):
-    """ids [T, K] int32 -> (offsets [E+1], pos [T*K], sorted_tok [T*K])."""
+def moe_align(ids, n_experts, weights=None):
+    """ids [T, K] int32 -> (offsets [E+1], pos [T*K], sorted_tok [T*K]); with ``weights`` (fp32 [T, K]) a fourth:
+    the pairs' weights in sorted order."""
     t, k = ids.shape
     if not ids.is_cuda:
         flat = ids.reshape(-1).long()
@@ -1078,14 +1080,19 @@ def moe_align(ids, n_experts):
         counts = torch.bincount(flat, minlength=n_experts)
         offsets = torch.zeros(n_experts + 1, dtype=torch.int32)
         offsets[1:] = counts.cumsum(0)
-        return offsets, pos.int(), (order // k).int()
+        out = (offsets, pos.int(), (order // k).int())
+        return out if weights is None else (*out, weights.reshape(-1)[order])
     offsets = torch.empty((n_experts + 1,), dtype=torch.int32, device=ids.device)
     pos = torch.empty((t * k,), dtype=torch.int32, device=ids.device)
     sorted_tok = torch.empty((t * k,), dtype=torch.int32, device=ids.device)
-    rc = _kernels().vpsa_moe_align(_p(ids.contiguous()), _p(offsets), _p(pos), _p(sorted_tok),
+    sorted_w = None
+    if weights is not None:
+        assert weights.dtype == torch.float32 and weights.is_contiguous() and weights.numel() == t * k
+        sorted_w = torch.empty((t * k,), dtype=torch.float32, device=ids.device)
+    rc = _kernels().vpsa_moe_align(_p(ids.contiguous()), _p(offsets), _p(pos), _p(sorted_tok), _p(weights), _p(sorted_w),
                                    c_int(t * k), c_int(n_experts), c_int(k), _stream())
     _check(rc, "moe_align")
-    return offsets, pos, sorted_tok
+    return (offsets, pos, sorted_tok) if weights is None else (offsets, pos, sorted_tok, sorted_w)
 
 
 def moe_permute(x, sorted_tok):
@@ -1196,7 +1203,7 @@ def tile_gemm_supported(n: int, k: int, silu_mul: bool = False) -> bool:
 
 
 def tile_gemm(a, w, offsets=None, rows=None, arow_idx=None, silu_mul=False, residual=None, out=None, glu_clamp=None,
-              relu_sq=False, xielu=None, gelu_mul=False):
+              relu_sq=False, xielu=None, gelu_mul=False, row_scale=None):
     """The prefill GEMM (``csrc/kernels/tile_gemm.hip``): out[r] = epilogue(a[arow_idx[r] or r] @ w[g]^T).
 
     a [*, K] bf16; w [N, K] (dense) or [G, N, K] (grouped, with offsets [G + 1] int32 ON THE DEVICE:
@@ -1206,7 +1213,8 @@ def tile_gemm(a, w, offsets=None, rows=None, arow_idx=None, silu_mul=False, resi
     rows] as for silu_mul, out = min(g, limit) * sigmoid(alpha min(g, limit)) * (clamp(u, +-limit) + bias).
     relu_sq: out = relu(product)^2.  xielu = (a_pos, a_neg): out = a_pos z^2 + z / 2 for z > 0, else
     a_neg (exp(z) - 1 - z) + z / 2.  gelu_mul: paired like silu_mul, out = gelu(gate) * up with gelu in its tanh
-    form.  Rows at or past offsets[G] are left unwritten."""
+    form.  row_scale (fp32 [rows], with glu_clamp): gate and up of an output row are multiplied by its factor before
+    the clamps.  Rows at or past offsets[G] are left unwritten."""
     paired = silu_mul or glu_clamp is not None or gelu_mul
     if w.dim() == 2:
         w = w.unsqueeze(0)
@@ -1216,6 +1224,8 @@ def tile_gemm(a, w, offsets=None, rows=None, arow_idx=None, silu_mul=False, resi
     n_out = n // 2 if paired else n
     _bf16_cuda(a, w, residual)
     assert w.is_contiguous() and a.stride(-1) == 1 and a.shape[1] == k
+    assert row_scale is None or (glu_clamp is not None and row_scale.is_cuda and row_scale.dtype == torch.float32
+                                 and row_scale.is_contiguous() and row_scale.numel() >= rows)
     assert sum((silu_mul, glu_clamp is not None, relu_sq, residual is not None, xielu is not None, gelu_mul)) <= 1
     if offsets is not None:
         assert offsets.dtype == torch.int32 and offsets.numel() == g + 1 and offsets.is_cuda
@@ -1237,7 +1247,7 @@ def tile_gemm(a, w, offsets=None, rows=None, arow_idx=None, silu_mul=False, resi
     rc = _kernels().vpsa_tile_gemm(_p(a), c_long(a.stride(0)), _p(arow_idx), _p(w), _p(offsets), c_int(g), _p(out),
                                    c_long(out.stride(0)), c_int(rows), c_int(n), c_int(k), c_int(epi), _p(residual),
                                    c_long(residual.stride(0) if residual is not None else 0), c_long(a.shape[0]),
-                                   c_float(lim), c_float(alpha), c_float(bias), _stream())
+                                   c_float(lim), c_float(alpha), c_float(bias), _p(row_scale), _stream())
     _check(rc, "tile_gemm")
     return out
 
@@ -1339,11 +1349,12 @@ def lora_expand(h, bs, slots, y, r_pad):
 
 # --------------------------------------------------------------------------- latent attention, group routing, fp32 residual
 from .latent import (add_rms_norm, build_latent_tiles, embed_scale, gate_up_glu_clamp, gather_rows, glu_clamp,  # noqa: E402,F401
+                     depth_mix_rms_norm, embed_rms_norm, moe_glu, poly_norm, soft_cap, up_poly_norm,
                      gate_up_act, gated_add_rms_norm, glu_act, rms_norm_add, route_softmax,
                      group_topk, latent_attention, moe_glu_grouped, moe_glu_grouped_supported, up_relu_sq,
                      latent_kv_write, latent_mfma_supported, latent_tile_kernel_takes, moe_finish, relu_sq, rms_norm_rows, rope_pairs, sigmoid_gate)
 
 # --------------------------------------------------------------------------- recurrent mixers, windowed attention, Dynamic Tanh
-from .seqmix import (add_dyt_norm, build_scan_pieces, build_window_tiles, head_rms_norm, mix_heads, recurrent_scan, short_conv_qkv,  # noqa: E402,F401
+from .seqmix import (add_dyt_norm, build_gru_pieces, build_scan_pieces, mingru_scan, build_window_tiles, head_rms_norm, mix_heads, recurrent_scan, short_conv_qkv,  # noqa: E402,F401
                      diff_heads, gla_prepare, head_finish, mlstm_prepare, pool_blocks, prepared_scan, qk_norm_write, scan_state_cols,
                      up_xielu, window_attention, window_cache_elems, window_decode_splits, window_mfma_supported, xielu)

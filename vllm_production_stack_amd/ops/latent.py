@@ -61,6 +61,24 @@ def embed_scale(ids, embed, scale: float):
     return out
 
 
+def embed_rms_norm(ids, embed, weight, eps: float, out=None):
+    """fp32 [T, width] = rmsnorm(embed[ids]) * weight; ``out`` (fp32, contiguous): a buffer that gets a second copy."""
+    if not embed.is_cuda:
+        y = reference.embed_rms_norm(ids, embed, weight, eps)
+        if out is not None:
+            out.copy_(y)
+        return y
+    o = _ops()
+    _f32(weight, out)
+    assert ids.dtype == torch.int64 and embed.is_contiguous() and weight.numel() == embed.shape[1]
+    y = torch.empty((ids.shape[0], embed.shape[1]), dtype=torch.float32, device=embed.device)
+    assert out is None or out.shape == y.shape
+    o._check(o._kernels().vpsa_embed_rmsnorm(o._p(ids), o._p(embed), o._p(weight), o._p(y), o._p(out), c_int(y.shape[0]),
+                                             c_int(y.shape[1]), c_float(eps), c_int(_dt(embed)), o._stream()),
+             "embed_rms_norm")
+    return y
+
+
 def add_rms_norm(residual, delta, weight, eps: float, out_dtype, want_out: bool = True):
     """residual (fp32, in place) += delta; returns rmsnorm(residual) * weight in ``out_dtype``."""
     if not residual.is_cuda:
@@ -111,6 +129,33 @@ def gated_add_rms_norm(residual, deltas, gate, gate_bias, weight, eps: float, ou
         c_long(d2.stride(0) if d2 is not None else 0), o._p(w2), c_float(c2), o._p(gate),
         c_long(gate.stride(0) if gate is not None else 0), o._p(gate_bias), o._p(extra), o._p(extra_vec), o._p(weight),
         o._p(y), c_int(t), c_int(n), c_float(eps), c_int(_DT[out_dtype]), o._stream()), "gated_add_rms_norm")
+    return y
+
+
+def depth_mix_rms_norm(residual, delta, delta_weight, history, n_prev: int, keep: bool, coef, weight, eps: float, out_dtype,
+                       want_out: bool = True):
+    """The end of a layer whose result joins a weighted average over the depth.  With s = residual + n(delta),
+    n(d) = rmsnorm(d) * ``delta_weight`` (None: d itself; ``delta`` None: s = residual), the layer's result:
+    history[n_prev] = s (``keep``), residual (fp32, in place) = sum_j coef[j] history[j], j < n_prev, + coef[n_prev] s.
+    ``history`` fp32 [*, T, n] holds the embedding output and the results of the layers before; ``coef`` fp32
+    [n_prev + 1]; the delta is in ``out_dtype`` or fp32 (a mixture's sum).  Returns rmsnorm(residual) * weight in
+    ``out_dtype`` (None without ``want_out``)."""
+    if not residual.is_cuda:
+        return reference.depth_mix_rms_norm(residual, delta, delta_weight, history, n_prev, keep, coef, weight, eps, out_dtype,
+                                            want_out)
+    o = _ops()
+    _f32(residual, delta_weight, history, coef, weight)
+    t, n = residual.shape
+    if t == 0:
+        return torch.empty((0, n), dtype=out_dtype, device=residual.device) if want_out else None
+    assert history.shape[1:] == (t, n) and history.shape[0] >= n_prev + (1 if keep else 0) and coef.numel() == n_prev + 1
+    assert delta is None or (_rows(delta) and delta.shape == (t, n) and delta.dtype in (out_dtype, torch.float32))
+    y = torch.empty((t, n), dtype=out_dtype, device=residual.device) if want_out else None
+    o._check(o._kernels().vpsa_depth_mix_rmsnorm(
+        o._p(residual), o._p(delta), c_long(delta.stride(0) if delta is not None else 0),
+        c_int(1 if (delta is not None and delta.dtype == torch.float32) else 0), o._p(delta_weight), o._p(history),
+        c_long(history.stride(0)), c_int(n_prev), c_int(1 if keep else 0), o._p(coef), o._p(weight), o._p(y), c_int(t),
+        c_int(n), c_float(eps), c_int(_DT[out_dtype]), o._stream()), "depth_mix_rms_norm")
     return y
 
 
@@ -300,15 +345,43 @@ def relu_sq(x):
     return y
 
 
-def glu_clamp(x, limit: float, alpha: float = 1.702, up_bias: float = 1.0):
-    """x [rows, 2 I] = gate | up  ->  min(g, limit) * sigmoid(alpha min(g, limit)) * (clamp(u, +-limit) + up_bias)."""
-    if not x.is_cuda:
-        return reference.glu_clamp(x, limit, alpha, up_bias)
+def poly_norm(z, act, eps: float):
+    """a N(z) + b N(z^2) + c N(z^3) + e over rows: powers element by element, N(v) = v / sqrt(mean(v^2) + eps) over the
+    row, (a, b, c, e) = ``act`` (fp32 [4] on the device)."""
+    if not z.is_cuda:
+        return reference.poly_norm(z, act, eps)
     o = _ops()
-    assert _rows(x) and x.shape[1] % 2 == 0
+    _f32(act)
+    assert _rows(z) and act.numel() == 4
+    y = torch.empty(z.shape, dtype=z.dtype, device=z.device)
+    o._check(o._kernels().vpsa_poly_norm(o._p(z), c_long(z.stride(0)), o._p(act), o._p(y), c_int(z.shape[0]),
+                                         c_int(z.shape[1]), c_float(eps), c_int(_dt(z)), o._stream()), "poly_norm")
+    return y
+
+
+def soft_cap(x, cap: float):
+    """fp32 cap * tanh(x / cap)."""
+    if not x.is_cuda:
+        return reference.soft_cap(x, cap)
+    o = _ops()
+    assert x.is_contiguous() and cap > 0
+    y = torch.empty(x.shape, dtype=torch.float32, device=x.device)
+    o._check(o._kernels().vpsa_soft_cap(o._p(x), o._p(y), c_long(x.numel()), c_float(cap), c_int(_dt(x)), o._stream()),
+             "soft_cap")
+    return y
+
+
+def glu_clamp(x, limit: float, alpha: float = 1.702, up_bias: float = 1.0, row_scale=None):
+    """x [rows, 2 I] = gate | up  ->  min(g, limit) * sigmoid(alpha min(g, limit)) * (clamp(u, +-limit) + up_bias).
+    ``row_scale`` (fp32 [rows]): g and u are multiplied by their row's factor first (a factor on the row's input)."""
+    if not x.is_cuda:
+        return reference.glu_clamp(x, limit, alpha, up_bias, row_scale)
+    o = _ops()
+    _f32(row_scale)
+    assert _rows(x) and x.shape[1] % 2 == 0 and (row_scale is None or row_scale.numel() == x.shape[0])
     inter = x.shape[1] // 2
     y = torch.empty((x.shape[0], inter), dtype=x.dtype, device=x.device)
-    o._check(o._kernels().vpsa_glu_clamp(o._p(x), c_long(x.stride(0)), o._p(y), c_int(x.shape[0]), c_int(inter),
+    o._check(o._kernels().vpsa_glu_clamp(o._p(x), c_long(x.stride(0)), o._p(row_scale), o._p(y), c_int(x.shape[0]), c_int(inter),
                                          c_float(limit), c_float(alpha), c_float(up_bias), c_int(_dt(x)), o._stream()),
              "glu_clamp")
     return y
@@ -405,8 +478,9 @@ def gather_rows(x, idx):
 
 
 def moe_finish(residual, y, weights, pos, shared=None, gate=None, overwrite: bool = False):
-    """residual fp32 [T, n] += sum_k weights[t, k] * y[pos[t * K + k]] (+ gate[t] * shared[t]).  ``overwrite``: the sum
-    replaces what ``residual`` held (a buffer that need not be cleared first)."""
+    """residual fp32 [T, n] += sum_k weights[t, k] * y[pos[t * K + k]] (+ gate[t] * shared[t]).  ``weights`` None: every
+    pair counts once (``pos`` then holds T * K entries).  ``overwrite``: the sum replaces what ``residual`` held (a
+    buffer that need not be cleared first)."""
     if not residual.is_cuda:
         if overwrite:
             residual.zero_()
@@ -415,8 +489,9 @@ def moe_finish(residual, y, weights, pos, shared=None, gate=None, overwrite: boo
     _f32(residual, weights, gate)
     t, n = residual.shape
     assert y.is_contiguous() and y.shape[1] == n and pos.dtype == torch.int32
+    topk = weights.shape[1] if weights is not None else pos.numel() // max(t, 1)
     assert shared is None or (shared.is_contiguous() and shared.shape == (t, n))
-    o._check(o._kernels().vpsa_moe_finish(o._p(residual), o._p(y), o._p(weights), o._p(pos), c_int(weights.shape[1]),
+    o._check(o._kernels().vpsa_moe_finish(o._p(residual), o._p(y), o._p(weights), o._p(pos), c_int(topk),
                                           o._p(shared), o._p(gate), c_int(t), c_int(n), c_int(1 if overwrite else 0),
                                           c_int(_dt(y, shared)), o._stream()), "moe_finish")
     return residual
@@ -441,20 +516,49 @@ def up_relu_sq(x, w_up):
     return relu_sq(o.linear(x, w_up))
 
 
+def up_poly_norm(x, w_up, act, eps: float):
+    """poly_norm(x @ W.T): the projection, then one pass over its rows (the norms need whole rows)."""
+    return poly_norm(_ops().linear(x, w_up), act, eps)
+
+
 def moe_glu_grouped_supported(x, w13, w2) -> bool:
     o = _ops()
     return (x.is_cuda and x.dtype == torch.bfloat16 and x.is_contiguous() and w13.is_contiguous() and w2.is_contiguous()
             and o.tile_gemm_supported(w13.shape[1], w13.shape[2], True) and o.tile_gemm_supported(w2.shape[1], w2.shape[2]))
 
 
-def moe_glu_grouped(x, w13, w2, ids, limit: float, alpha: float = 1.702, up_bias: float = 1.0):
+def moe_glu(x, w13, w2, ids, limit: float, alpha: float = 1.702, up_bias: float = 1.0, scale=None):
+    """Clamped gated units of a mixture over its (token, unit) pairs: ``moe_glu_grouped`` where its kernels tile the
+    shape, else (the CPU, fp32, other widths) unit by unit on the sorted rows, which reads the row counts on the host.
+    ``scale`` fp32 [T, K]: a pair's unit sees its token's row times the pair's factor.
+    Returns (y [T * K, hidden] in sorted order, pos [T * K]: the sorted row of pair t * K + k)."""
+    if moe_glu_grouped_supported(x, w13, w2):
+        return moe_glu_grouped(x, w13, w2, ids, limit, alpha, up_bias, scale)
+    o = _ops()
+    t, k = ids.shape
+    offsets, pos, sorted_tok, *sw = o.moe_align(ids, w13.shape[0], scale)
+    xs = gather_rows(x, sorted_tok)
+    ys = torch.empty((t * k, x.shape[1]), dtype=x.dtype, device=x.device)
+    off = offsets.tolist()
+    for e in range(w13.shape[0]):
+        a, b = off[e], off[e + 1]
+        if b > a:
+            act = glu_clamp(torch.nn.functional.linear(xs[a:b], w13[e]), limit, alpha, up_bias,
+                            row_scale=sw[0][a:b] if sw else None)
+            torch.matmul(act, w2[e].t(), out=ys[a:b])
+    return ys, pos
+
+
+def moe_glu_grouped(x, w13, w2, ids, limit: float, alpha: float = 1.702, up_bias: float = 1.0, scale=None):
     """Clamped gated units of a mixture over the device-sorted (token, unit) pairs: two grouped
     matrix-core GEMMs (the first gathers its token rows and applies the activation in its epilogue).
-    The host never reads the per-unit counts: no synchronisation, HIP-graph capturable.
+    ``scale`` fp32 [T, K]: a pair's unit sees its token's row times the pair's factor (applied to gate and up in the
+    epilogue).  The host never reads the per-unit counts: no synchronisation, HIP-graph capturable.
     Returns (y [T * K, hidden] in sorted order, pos [T * K]: the sorted row of pair t * K + k)."""
     o = _ops()
     t, k = ids.shape
-    offsets, pos, sorted_tok = o.moe_align(ids, w13.shape[0])
+    offsets, pos, sorted_tok, *sw = o.moe_align(ids, w13.shape[0], scale)
+    sw = sw[0] if sw else None
     hidden, inter = x.shape[1], w2.shape[2]
     if t <= o.MOE_MFMA_MAX_TOKENS and o.moe_mfma_supported(hidden, inter) and limit > 0:
         # decode-sized batches: each routed unit's weights streamed once against its few tokens
@@ -466,5 +570,5 @@ def moe_glu_grouped(x, w13, w2, ids, limit: float, alpha: float = 1.702, up_bias
                                                 c_int(inter), c_float(limit), c_float(alpha), c_float(up_bias),
                                                 o._stream()), "moe_mfma_act")
         return y, pos
-    act = o.tile_gemm(x, w13, offsets, rows=t * k, arow_idx=sorted_tok, glu_clamp=(limit, alpha, up_bias))
+    act = o.tile_gemm(x, w13, offsets, rows=t * k, arow_idx=sorted_tok, glu_clamp=(limit, alpha, up_bias), row_scale=sw)
     return o.tile_gemm(act, w2, offsets, rows=t * k), pos

@@ -353,6 +353,11 @@ def embed_scale(ids, embed, scale):
     return embed[ids.long()].float() * scale
 
 
+def embed_rms_norm(ids, embed, weight, eps):
+    e = embed[ids.long()].float()
+    return e * torch.rsqrt(e.pow(2).mean(-1, keepdim=True) + eps) * weight
+
+
 def add_rms_norm(residual, delta, weight, eps, out_dtype, want_out=True):
     if delta is not None:
         residual.add_(delta.float())
@@ -380,6 +385,35 @@ def gated_add_rms_norm(residual, deltas, gate, gate_bias, extra, extra_vec, weig
     if not want_out:
         return None
     return (residual * torch.rsqrt(residual.pow(2).mean(-1, keepdim=True) + eps) * weight).to(out_dtype)
+
+
+def depth_mix_rms_norm(residual, delta, delta_weight, history, n_prev, keep, coef, weight, eps, out_dtype, want_out=True):
+    if delta is not None:
+        d = delta.float()
+        if delta_weight is not None:
+            d = d * torch.rsqrt(d.pow(2).mean(-1, keepdim=True) + eps) * delta_weight
+        residual.add_(d)
+    if keep:
+        history[n_prev].copy_(residual)
+    residual.mul_(coef[n_prev])
+    for j in range(n_prev):
+        residual.add_(history[j] * coef[j])
+    if not want_out:
+        return None
+    return (residual * torch.rsqrt(residual.pow(2).mean(-1, keepdim=True) + eps) * weight).to(out_dtype)
+
+
+def poly_norm(z, act, eps):
+    zf = z.float()
+    total = act[3]
+    for k in range(3):
+        p = zf ** (k + 1)
+        total = total + act[k] * p * torch.rsqrt(p.pow(2).mean(-1, keepdim=True) + eps)
+    return total.to(z.dtype)
+
+
+def soft_cap(x, cap):
+    return cap * torch.tanh(x.float() / cap)
 
 
 def rms_norm_add(residual, delta, weight, eps, out_dtype, want_out=True):
@@ -488,10 +522,11 @@ def relu_sq(x):
     return torch.relu(x.float()).pow(2).to(x.dtype)
 
 
-def glu_clamp(x, limit, alpha, up_bias):
+def glu_clamp(x, limit, alpha, up_bias, row_scale=None):
     inter = x.shape[-1] // 2
-    g = x[..., :inter].float().clamp(max=limit)
-    u = x[..., inter:].float().clamp(-limit, limit)
+    xf = x.float() if row_scale is None else x.float() * row_scale[:, None]
+    g = xf[..., :inter].clamp(max=limit)
+    u = xf[..., inter:].clamp(-limit, limit)
     return (g * torch.sigmoid(alpha * g) * (u + up_bias)).to(x.dtype)
 
 
@@ -516,6 +551,8 @@ def group_topk(logits, experts, groups, keep, topk, route_scale, extra, normaliz
 
 
 def moe_finish(residual, y, weights, pos, shared, gate):
+    if weights is None:
+        weights = torch.ones((residual.shape[0], pos.numel() // max(residual.shape[0], 1)))
     t, k = weights.shape
     if k:  # a pair of weight 0 is skipped, as in the kernel: its row of y may never have been written
         rows = torch.where((weights != 0)[:, :, None], y[pos.long()].view(t, k, -1).float(), 0.0)
@@ -640,6 +677,27 @@ def prepared_scan(prep, proj, v_col, heads, dim, vdim, cols, unit_col, state, st
             S.mul_(prep[r, :, 2].unsqueeze(-1)).add_(prep[r, :, 1].unsqueeze(-1) * v[r].unsqueeze(1))
             out[r] = torch.einsum("hdv,hd->hv", S, prep[r, :, 0])
     return out
+
+
+def mingru_scan(z, x, g, z_bias, x_bias, state, state_off, seq_cu, seq_state, positions):
+    t, n = z.shape
+    zz = torch.sigmoid(z.float() + z_bias)
+    u = x.float() + x_bias
+    cand = torch.where(u >= 0, u + 0.5, torch.sigmoid(u))
+    out = torch.empty((t, n), dtype=torch.float32)
+    cu = seq_cu.tolist()
+    for i, slot in enumerate(seq_state.tolist()):
+        a, b = cu[i], cu[i + 1]
+        if a == b:
+            continue
+        fresh = slot < 0 or int(positions[a]) == 0
+        s = torch.zeros(n) if fresh else state[slot, state_off:state_off + n].clone()
+        for r in range(a, b):
+            s = (1 - zz[r]) * s + zz[r] * cand[r]
+            out[r] = s
+        if slot >= 0:
+            state[slot, state_off:state_off + n] = s
+    return (out * torch.nn.functional.silu(g.float())).to(z.dtype)
 
 
 def head_finish(o, eps, out_dtype, vdim, stab, unit, weight, gate, gate_act):

@@ -266,6 +266,62 @@ def prepared_scan(prep, proj, v_col: int, heads: int, dim: int, vdim: int, state
     return out
 
 
+GRU_PIECE_ROWS = 128        # rows of a piece of a minGRU walk (what a workgroup holds in registers)
+GRU_PIECE_MIN_ROWS = 257    # sequences of a step shorter than this are walked in one go
+
+
+def build_gru_pieces(q_lens):
+    """Cuts the sequences of a step into pieces for ``mingru_scan`` (arrays as for ``build_scan_pieces``), or None
+    when no sequence is long enough to pay for the second pass."""
+    import numpy as np
+
+    if not q_lens or max(q_lens) < GRU_PIECE_MIN_ROWS:
+        return None
+    lens = np.asarray(q_lens, dtype=np.int64)
+    counts = (lens + GRU_PIECE_ROWS - 1) // GRU_PIECE_ROWS
+    first = np.concatenate([[0], np.cumsum(counts)])
+    seq = np.repeat(np.arange(len(lens)), counts)
+    at = (np.arange(first[-1]) - first[seq]) * GRU_PIECE_ROWS   # a piece's first row within its sequence
+    row = (np.cumsum(lens) - lens)[seq] + at
+    pieces = np.stack([seq, row, np.minimum(GRU_PIECE_ROWS, lens[seq] - at)], axis=1)
+    return np.ascontiguousarray(pieces, dtype=np.int32), first.astype(np.int32)
+
+
+def mingru_scan(proj, z_col: int, x_col: int, g_col: int, width: int, z_bias, x_bias, state, state_off: int, seq_cu,
+                seq_state, positions, pieces=None):
+    """A gated recurrence whose gates read the current token only, channel by channel over each sequence's rows:
+    z = sigmoid(pz + z_bias), u = px + x_bias, cand = u + 1/2 where u >= 0 else sigmoid(u),
+    S <- (1 - z) S + z cand, y = S * silu(pg), with pz, px and pg column ranges of ``proj`` [T, cols] (activation
+    dtype), the biases fp32 [width] and S (fp32) carried in the sequence's state slot.  ``pieces``: device copies of
+    ``build_gru_pieces`` for steps with long chunks.  Returns y [T, width] in the activation dtype."""
+    cols = [proj[:, c:c + width] for c in (z_col, x_col, g_col)]
+    if not proj.is_cuda:
+        return reference.mingru_scan(*cols, z_bias, x_bias, state, state_off, seq_cu, seq_state, positions)
+    o = _ops()
+    _f32(z_bias, x_bias, state)
+    _i32(seq_cu, seq_state, positions)
+    t = proj.shape[0]
+    assert _rows(proj) and max(z_col, x_col, g_col) + width <= proj.shape[1] and z_bias.numel() == x_bias.numel() == width
+    assert state_off + width <= state.shape[1] and seq_cu.numel() == seq_state.numel() + 1 and positions.numel() >= t
+    y = torch.empty((t, width), dtype=proj.dtype, device=proj.device)
+    pc = sp = ws = start = None
+    n_pieces = 0
+    n_seqs = seq_state.numel()
+    if pieces is not None:
+        pc, sp = pieces
+        _i32(pc, sp)
+        n_pieces = pc.shape[0]
+        assert pc.shape[1] == 3 and sp.numel() == seq_cu.numel()
+        ws = torch.empty((2, n_pieces, width), dtype=torch.float32, device=proj.device)
+        start = torch.empty((n_seqs, width), dtype=torch.float32, device=proj.device)
+    o._check(o._kernels().vpsa_mingru(
+        *[o._p(c) for c in cols], c_long(proj.stride(0)), c_int(width), o._p(z_bias), o._p(x_bias), _at(state, state_off),
+        c_long(state.stride(0)), o._p(seq_cu), o._p(seq_state), c_int(n_seqs), o._p(positions), o._p(y), c_int(t), o._p(pc),
+        o._p(sp), c_int(n_pieces), o._p(ws[0] if ws is not None else None), o._p(ws[1] if ws is not None else None),
+        o._p(start), c_int(_dt(proj)), o._stream()), "mingru_scan")
+    return y
+
+
 GATE_ACTS = {"silu": 0, "sigmoid": 1}
 
 
