@@ -1,6 +1,6 @@
 """Prefill and decode throughput of one decoder design beside the closest existing one at equal size.
 
-    python bench.py --arch-compare zururax|revelix|pelatar|zetalorn [--arch-sizes s,m] [--arch-prompt 4096] [--arch-batch 32]
+    python bench.py --arch-compare zururax|revelix|pelatar|zetalorn|zupilorn [--arch-sizes s,m] [--arch-prompt 4096] [--arch-batch 32]
 
 Random weights at layer shapes of real models (a few layers each); both models run through the same
 engine (scheduler, paged pool, HIP-graph decode).  Prefill: prompts of --arch-prompt tokens in chunks of
@@ -34,6 +34,8 @@ def _configs(design: str, size: str):
         return _pelatar_configs(size)
     if design == "zetalorn":
         return _zetalorn_configs(size)
+    if design == "zupilorn":
+        return _zupilorn_configs(size)
     if design != "zururax":
         raise SystemExit(f"--arch-compare: unknown design {design!r}")
 
@@ -119,6 +121,21 @@ def _zetalorn_configs(size: str):
                           zetalorn_stack(z["width"], z["heads"], z["experts"], z["ff"], z["top"]),
                           loop={"start": 0, "stop": 2, "times": 2}, logit_scale=0.5, max_position_embeddings=32768)
     return new, _pelatar_configs(size)[0]
+
+
+def _zupilorn_configs(size: str):
+    """Zupilorn (latent attention with a dense PolyNorm feed-forward and a minGRU as wide as the model with routed
+    clamped units, in turn; every layer's result in the depth average) beside the closest existing design, Zururax at
+    the same width, depth, head shapes, latent rank, units and dense feed-forward: its attention runs the same kernels
+    over the same cache entries, its routed units the same grouped GEMMs."""
+    from vllm_production_stack_amd.engine.config import zupilorn_config, zupilorn_stack
+
+    z = SIZES[size]
+    ff = z["top"] * z["ff"] + z["shared"]
+    new = zupilorn_config(f"zupilorn-{size}", VOCAB, z["width"],
+                          zupilorn_stack(z["width"], z["heads"], ff, z["experts"], z["ff"], z["top"], blocks=z["layers"] // 2),
+                          logit_softcap=30.0, max_position_embeddings=32768)
+    return new, _configs("zururax", size)[0]
 
 
 def _measure(cfg, a) -> dict:

@@ -24,7 +24,7 @@
 //   depth_mix_rmsnorm  s = residual + n(delta) is a layer's result, kept in the history of layer results;
 //                      residual = sum_j a_j history_j + a_last s;  y = rmsnorm(residual) w
 //   poly_norm          y = a N(z) + b N(z^2) + c N(z^3) + e, N = division by the row's root mean square
-//   soft_cap           y = cap tanh(x / cap)                                             (fp32 out)
+//   soft_cap           y = cap tanh(x / cap)
 //   glu_act            silu(g) * u  or  gelu_tanh(g) * u  of  x = g | u
 //   gather_rows        xs[r] = x[idx[r]]
 //   moe_finish         residual[t] += sum_k w[t,k] * y[pos[t,k]] + gate[t] * shared[t]   (w optional: all 1)
@@ -813,10 +813,10 @@ __global__ __launch_bounds__(256) void poly_norm_kernel(const T* __restrict__ z,
 }
 
 template <typename T>
-__global__ __launch_bounds__(256) void soft_cap_kernel(const T* __restrict__ x, float* __restrict__ y, long n, float cap) {
+__global__ __launch_bounds__(256) void soft_cap_kernel(const T* __restrict__ x, T* __restrict__ y, long n, float cap) {
   const float inv = 1.f / cap;
   for (long i = blockIdx.x * 256L + threadIdx.x; i < n; i += (long)gridDim.x * 256)
-    y[i] = cap * tanhf(Conv<T>::ld(x + i) * inv);
+    Conv<T>::st(y + i, cap * tanhf(Conv<T>::ld(x + i) * inv));
 }
 
 // x [rows, 2 inter] = gate | up  ->  act(gate) * up;  kind 0: silu, 1: gelu in its tanh form
@@ -1078,12 +1078,12 @@ VPSA_EXPORT int vpsa_poly_norm(const void* z, long z_stride, const float* act, v
   return 0;
 }
 
-VPSA_EXPORT int vpsa_soft_cap(const void* x, float* y, long n, float cap, int dtype, hipStream_t st) {
+VPSA_EXPORT int vpsa_soft_cap(const void* x, void* y, long n, float cap, int dtype, hipStream_t st) {
   if (n <= 0) return 0;
   if (!(cap > 0.f)) return -1;
   DISPATCH(dtype,
-           hipLaunchKernelGGL(soft_cap_kernel<bf16_t>, dim3(flat_grid(n)), dim3(256), 0, st, (const bf16_t*)x, y, n, cap),
-           hipLaunchKernelGGL(soft_cap_kernel<float>, dim3(flat_grid(n)), dim3(256), 0, st, (const float*)x, y, n, cap));
+           hipLaunchKernelGGL(soft_cap_kernel<bf16_t>, dim3(flat_grid(n)), dim3(256), 0, st, (const bf16_t*)x, (bf16_t*)y, n, cap),
+           hipLaunchKernelGGL(soft_cap_kernel<float>, dim3(flat_grid(n)), dim3(256), 0, st, (const float*)x, (float*)y, n, cap));
   return 0;
 }
 

@@ -360,12 +360,12 @@ def poly_norm(z, act, eps: float):
 
 
 def soft_cap(x, cap: float):
-    """fp32 cap * tanh(x / cap)."""
+    """cap * tanh(x / cap), computed in fp32, in x's dtype."""
     if not x.is_cuda:
         return reference.soft_cap(x, cap)
     o = _ops()
     assert x.is_contiguous() and cap > 0
-    y = torch.empty(x.shape, dtype=torch.float32, device=x.device)
+    y = torch.empty_like(x)
     o._check(o._kernels().vpsa_soft_cap(o._p(x), o._p(y), c_long(x.numel()), c_float(cap), c_int(_dt(x)), o._stream()),
              "soft_cap")
     return y
@@ -568,7 +568,7 @@ def moe_glu_grouped(x, w13, w2, ids, limit: float, alpha: float = 1.702, up_bias
         o._check(o._kernels().vpsa_moe_mfma_act(o._p(x), o._p(w13), o._p(w2), o._p(offsets), o._p(sorted_tok), o._p(act),
                                                 o._p(y), c_int(t), c_int(k), c_int(w13.shape[0]), c_int(hidden),
                                                 c_int(inter), c_float(limit), c_float(alpha), c_float(up_bias),
-                                                o._stream()), "moe_mfma_act")
+                                                o._p(sw), o._stream()), "moe_mfma_act")
         return y, pos
     act = o.tile_gemm(x, w13, offsets, rows=t * k, arow_idx=sorted_tok, glu_clamp=(limit, alpha, up_bias), row_scale=sw)
     return o.tile_gemm(act, w2, offsets, rows=t * k), pos

@@ -413,7 +413,7 @@ def poly_norm(z, act, eps):
 
 
 def soft_cap(x, cap):
-    return cap * torch.tanh(x.float() / cap)
+    return (cap * torch.tanh(x.float() / cap)).to(x.dtype)
 
 
 def rms_norm_add(residual, delta, weight, eps, out_dtype, want_out=True):
