@@ -8,7 +8,7 @@
 //   add_rmsnorm        residual += delta;  y = residual * rsqrt(mean(residual^2) + eps) * w
 //   rmsnorm_rows       y = x * rsqrt(mean(x^2) + eps) * w over a column range of a wider row
 //   latent_kv_write    a token's compressed KV entry: RMS-normed latent | rotated shared key part
-//                      -> paged cache row [rank + rot]
+//                      -> paged cache row [rank + rot]; optionally the rotation of the query heads as well
 //   rope_pairs         interleaved-pair rotary embedding of a column range of every head, in place
 //   latent_attention   causal attention of query rows in latent space over the paged entries with an
 //                      optional per-head sink logit in the softmax denominator
@@ -66,6 +66,26 @@ __device__ __forceinline__ float block_max(float v, float* red) {
   return s;
 }
 
+// 8 neighbouring values on 16-byte boundaries
+__device__ __forceinline__ void ld8(const float* p, float* v) {
+  const f32x4 a = *reinterpret_cast<const f32x4*>(p), b = *reinterpret_cast<const f32x4*>(p + 4);
+#pragma unroll
+  for (int e = 0; e < 4; ++e) v[e] = a[e], v[4 + e] = b[e];
+}
+__device__ __forceinline__ void ld8(const bf16_t* p, float* v) {
+  const u32x4 a = *reinterpret_cast<const u32x4*>(p);
+#pragma unroll
+  for (int e = 0; e < 4; ++e) v[2 * e] = bf16lo(a[e]), v[2 * e + 1] = bf16hi(a[e]);
+}
+__device__ __forceinline__ void st8(float* p, const float* v) {
+  *reinterpret_cast<f32x4*>(p) = (f32x4){v[0], v[1], v[2], v[3]};
+  *reinterpret_cast<f32x4*>(p + 4) = (f32x4){v[4], v[5], v[6], v[7]};
+}
+__device__ __forceinline__ void st8(bf16_t* p, const float* v) {
+  *reinterpret_cast<u32x4*>(p) = (u32x4){pack_bf16x2(v[0], v[1]), pack_bf16x2(v[2], v[3]), pack_bf16x2(v[4], v[5]),
+                                         pack_bf16x2(v[6], v[7])};
+}
+
 __device__ __forceinline__ float sigmoidf(float x) { return 1.f / (1.f + expf(-x)); }
 
 // ---------------------------------------------------------------------------------
@@ -78,7 +98,8 @@ __global__ __launch_bounds__(256) void embed_scale_kernel(const long* __restrict
   for (int i = threadIdx.x; i < width; i += 256) o[i] = Conv<T>::ld(e + i) * scale;
 }
 
-template <typename T>
+// V: rows of whole runs of 8 values on 16-byte boundaries
+template <typename T, bool V>
 __global__ __launch_bounds__(256) void embed_rmsnorm_kernel(const long* __restrict__ ids, const T* __restrict__ embed,
                                                             const float* __restrict__ w, float* __restrict__ out,
                                                             float* __restrict__ out2, int width, float eps) {
@@ -86,15 +107,36 @@ __global__ __launch_bounds__(256) void embed_rmsnorm_kernel(const long* __restri
   const long row = blockIdx.x;
   const T* e = embed + ids[row] * (long)width;
   float ss = 0.f;
-  for (int i = threadIdx.x; i < width; i += 256) {
-    const float v = Conv<T>::ld(e + i);
-    ss += v * v;
+  if constexpr (V) {
+    for (int i = threadIdx.x * 8; i < width; i += 2048) {
+      float v[8];
+      ld8(e + i, v);
+#pragma unroll
+      for (int k = 0; k < 8; ++k) ss += v[k] * v[k];
+    }
+  } else {
+    for (int i = threadIdx.x; i < width; i += 256) {
+      const float v = Conv<T>::ld(e + i);
+      ss += v * v;
+    }
   }
   const float inv = 1.f / sqrtf(block_sum(ss, red) / (float)width + eps);
-  for (int i = threadIdx.x; i < width; i += 256) {
-    const float v = Conv<T>::ld(e + i) * inv * w[i];
-    out[row * width + i] = v;
-    if (out2) out2[row * width + i] = v;
+  if constexpr (V) {
+    for (int i = threadIdx.x * 8; i < width; i += 2048) {
+      float v[8], g[8];
+      ld8(e + i, v);
+      ld8(w + i, g);
+#pragma unroll
+      for (int k = 0; k < 8; ++k) v[k] *= inv * g[k];
+      st8(out + row * width + i, v);
+      if (out2) st8(out2 + row * width + i, v);
+    }
+  } else {
+    for (int i = threadIdx.x; i < width; i += 256) {
+      const float v = Conv<T>::ld(e + i) * inv * w[i];
+      out[row * width + i] = v;
+      if (out2) out2[row * width + i] = v;
+    }
   }
 }
 
@@ -147,6 +189,7 @@ __global__ __launch_bounds__(256) void rmsnorm_rows_kernel(const T* __restrict__
 // [rank, rank + rot) are the shared key part, whose first rot_dims columns rotate in interleaved
 // pairs (2i, 2i+1) by the angle table cos_sin[pos] = cos[0 .. rot_dims/2) | sin[0 .. rot_dims/2).
 // The entry goes to cache + (slot / 64) * page_stride + (slot % 64) * (rank + rot); slot < 0 skips.
+// With q [rows, heads, *]: columns [q_col, q_col + rot_dims) of every query head turn by the same angles, in place.
 template <typename T>
 __global__ __launch_bounds__(256) void latent_kv_write_kernel(const T* __restrict__ x, long x_stride,
                                                               const float* __restrict__ w,
@@ -154,10 +197,23 @@ __global__ __launch_bounds__(256) void latent_kv_write_kernel(const T* __restric
                                                               const long* __restrict__ slots,
                                                               const float* __restrict__ cos_sin, T* __restrict__ cache,
                                                               long page_stride, int rank, int rot, int rot_dims,
-                                                              float eps) {
+                                                              float eps, T* __restrict__ q, long q_row, long q_head,
+                                                              int heads, int q_col) {
   __shared__ float red[4];
   const long row = blockIdx.x;
   const long slot = slots[row];
+  const int half = rot_dims >> 1;
+  const float* cs = cos_sin + (long)positions[row] * rot_dims;
+  if (q) {
+    for (int i = threadIdx.x; i < heads * half; i += 256) {
+      const int h = i / half, j = i % half;
+      T* p = q + row * q_row + h * q_head + q_col + 2 * j;
+      const float u = Conv<T>::ld(p), v = Conv<T>::ld(p + 1);
+      const float c = cs[j], s = cs[half + j];
+      Conv<T>::st(p, u * c - v * s);
+      Conv<T>::st(p + 1, v * c + u * s);
+    }
+  }
   if (slot < 0) return;
   const T* xr = x + row * x_stride;
   T* dst = cache + (slot / PAGE) * page_stride + (slot % PAGE) * (long)(rank + rot);
@@ -168,8 +224,6 @@ __global__ __launch_bounds__(256) void latent_kv_write_kernel(const T* __restric
   }
   const float inv = 1.f / sqrtf(block_sum(ss, red) / (float)rank + eps);
   for (int i = threadIdx.x; i < rank; i += 256) Conv<T>::st(dst + i, Conv<T>::ld(xr + i) * inv * w[i]);
-  const int half = rot_dims >> 1;
-  const float* cs = cos_sin + (long)positions[row] * rot_dims;
   for (int i = threadIdx.x; i < half; i += 256) {
     const float u = Conv<T>::ld(xr + rank + 2 * i), v = Conv<T>::ld(xr + rank + 2 * i + 1);
     const float c = cs[i], s = cs[half + i];
@@ -477,25 +531,6 @@ __global__ __launch_bounds__(256) void rmsnorm_add_kernel(float* __restrict__ re
 // with n_i(d) = rmsnorm(d) w_i where a weight w_i is given and d itself otherwise.  Every part is optional: no gate
 // means a plain add, no deltas only the extras (a second stream that re-enters, a vector per pass of a layer loop).
 // d1 in D (the activation dtype, or fp32 for a mixture's sum), d2, gate and y in T.
-__device__ __forceinline__ void ld8(const float* p, float* v) {
-  const f32x4 a = *reinterpret_cast<const f32x4*>(p), b = *reinterpret_cast<const f32x4*>(p + 4);
-#pragma unroll
-  for (int e = 0; e < 4; ++e) v[e] = a[e], v[4 + e] = b[e];
-}
-__device__ __forceinline__ void ld8(const bf16_t* p, float* v) {
-  const u32x4 a = *reinterpret_cast<const u32x4*>(p);
-#pragma unroll
-  for (int e = 0; e < 4; ++e) v[2 * e] = bf16lo(a[e]), v[2 * e + 1] = bf16hi(a[e]);
-}
-__device__ __forceinline__ void st8(float* p, const float* v) {
-  *reinterpret_cast<f32x4*>(p) = (f32x4){v[0], v[1], v[2], v[3]};
-  *reinterpret_cast<f32x4*>(p + 4) = (f32x4){v[4], v[5], v[6], v[7]};
-}
-__device__ __forceinline__ void st8(bf16_t* p, const float* v) {
-  *reinterpret_cast<u32x4*>(p) = (u32x4){pack_bf16x2(v[0], v[1]), pack_bf16x2(v[2], v[3]), pack_bf16x2(v[4], v[5]),
-                                         pack_bf16x2(v[6], v[7])};
-}
-
 // K > 0: rows of up to 2048 K values, a multiple of 8, every operand on 16-byte boundaries: a thread owns runs of 8
 // neighbouring values, loads every operand once with 16-byte loads and keeps the new stream in registers.
 // K = 0: any width and alignment, value by value, operands read again where needed.
@@ -843,7 +878,8 @@ __global__ __launch_bounds__(256) void gather_rows_kernel(const T* __restrict__ 
   for (int i = threadIdx.x; i < n; i += 256) xs[row * n + i] = src[i];
 }
 
-template <typename T>
+// V: rows of whole runs of 8 values on 16-byte boundaries
+template <typename T, bool V>
 __global__ __launch_bounds__(256) void moe_finish_kernel(float* __restrict__ residual, const T* __restrict__ y,
                                                          const float* __restrict__ weights,
                                                          const int* __restrict__ pos, int topk,
@@ -862,17 +898,50 @@ __global__ __launch_bounds__(256) void moe_finish_kernel(float* __restrict__ res
     wk[k] = k < topk ? (weights ? weights[t * topk + k] : 1.f) : 0.f;
     yk[k] = y + (long)(wk[k] != 0.f ? pos[t * topk + k] : 0) * n;
   }
-  for (int i = threadIdx.x; i < n; i += 256) {
-    float a = 0.f;
+  constexpr int W = V ? 8 : 1;
+  auto ld = [](const T* p, float* v) {
+    if constexpr (V) ld8(p, v);
+    else v[0] = Conv<T>::ld(p);
+  };
+  for (int i = (blockIdx.y * 256 + threadIdx.x) * W; i < n; i += gridDim.y * 256 * W) {
+    float a[W];
+#pragma unroll
+    for (int e = 0; e < W; ++e) a[e] = 0.f;
 #pragma unroll
     for (int k = 0; k < AHEAD; ++k)
-      if (wk[k] != 0.f) a += wk[k] * Conv<T>::ld(yk[k] + i);
+      if (wk[k] != 0.f) {
+        float v[W];
+        ld(yk[k] + i, v);
+#pragma unroll
+        for (int e = 0; e < W; ++e) a[e] += wk[k] * v[e];
+      }
     for (int k = AHEAD; k < topk; ++k) {
       const float w = weights ? weights[t * topk + k] : 1.f;
-      if (w != 0.f) a += w * Conv<T>::ld(y + (long)pos[t * topk + k] * n + i);
+      if (w != 0.f) {
+        float v[W];
+        ld(y + (long)pos[t * topk + k] * n + i, v);
+#pragma unroll
+        for (int e = 0; e < W; ++e) a[e] += w * v[e];
+      }
     }
-    if (shared) a += sg * Conv<T>::ld(shared + t * n + i);
-    residual[t * n + i] = overwrite ? a : residual[t * n + i] + a;
+    if (shared) {
+      float v[W];
+      ld(shared + t * n + i, v);
+#pragma unroll
+      for (int e = 0; e < W; ++e) a[e] += sg * v[e];
+    }
+    float* r = residual + t * n + i;
+    if constexpr (V) {
+      if (!overwrite) {
+        float v[8];
+        ld8(r, v);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) a[e] += v[e];
+      }
+      st8(r, a);
+    } else {
+      *r = overwrite ? a[0] : *r + a[0];
+    }
   }
 }
 
@@ -903,9 +972,10 @@ VPSA_EXPORT int vpsa_embed_scale(const long* ids, const void* embed, float* out,
 VPSA_EXPORT int vpsa_embed_rmsnorm(const long* ids, const void* embed, const float* w, float* out, float* out2, int rows,
                                    int width, float eps, int dtype, hipStream_t st) {
   if (rows <= 0) return 0;
-  DISPATCH(dtype,
-           hipLaunchKernelGGL(embed_rmsnorm_kernel<bf16_t>, dim3(rows), dim3(256), 0, st, ids, (const bf16_t*)embed, w, out, out2, width, eps),
-           hipLaunchKernelGGL(embed_rmsnorm_kernel<float>, dim3(rows), dim3(256), 0, st, ids, (const float*)embed, w, out, out2, width, eps));
+  const bool vec = width % 8 == 0 && (((uintptr_t)embed | (uintptr_t)w | (uintptr_t)out | (uintptr_t)out2) & 15) == 0;
+#define EN(T, V) embed_rmsnorm_kernel<T, V><<<rows, 256, 0, st>>>(ids, (const T*)embed, w, out, out2, width, eps)
+  DISPATCH(dtype, if (vec) EN(bf16_t, true); else EN(bf16_t, false), if (vec) EN(float, true); else EN(float, false));
+#undef EN
   return 0;
 }
 
@@ -929,13 +999,13 @@ VPSA_EXPORT int vpsa_rmsnorm_rows(const void* x, long x_stride, const float* w, 
 
 VPSA_EXPORT int vpsa_latent_kv_write(const void* x, long x_stride, const float* w, const int* positions,
                                      const long* slots, const float* cos_sin, void* cache, long page_stride,
-                                     int rows, int rank, int rot, int rot_dims, float eps, int dtype,
-                                     hipStream_t st) {
+                                     int rows, int rank, int rot, int rot_dims, float eps, void* q, long q_row,
+                                     long q_head, int heads, int q_col, int dtype, hipStream_t st) {
   if (rows <= 0) return 0;
   if (rot_dims > rot || (rot_dims & 1)) return -1;
   DISPATCH(dtype,
-           hipLaunchKernelGGL(latent_kv_write_kernel<bf16_t>, dim3(rows), dim3(256), 0, st, (const bf16_t*)x, x_stride, w, positions, slots, cos_sin, (bf16_t*)cache, page_stride, rank, rot, rot_dims, eps),
-           hipLaunchKernelGGL(latent_kv_write_kernel<float>, dim3(rows), dim3(256), 0, st, (const float*)x, x_stride, w, positions, slots, cos_sin, (float*)cache, page_stride, rank, rot, rot_dims, eps));
+           hipLaunchKernelGGL(latent_kv_write_kernel<bf16_t>, dim3(rows), dim3(256), 0, st, (const bf16_t*)x, x_stride, w, positions, slots, cos_sin, (bf16_t*)cache, page_stride, rank, rot, rot_dims, eps, (bf16_t*)q, q_row, q_head, heads, q_col),
+           hipLaunchKernelGGL(latent_kv_write_kernel<float>, dim3(rows), dim3(256), 0, st, (const float*)x, x_stride, w, positions, slots, cos_sin, (float*)cache, page_stride, rank, rot, rot_dims, eps, (float*)q, q_row, q_head, heads, q_col));
   return 0;
 }
 
@@ -1139,8 +1209,13 @@ VPSA_EXPORT int vpsa_moe_finish(float* residual, const void* y, const float* wei
                                 const void* shared, const float* gate, int tokens, int n, int overwrite, int dtype,
                                 hipStream_t st) {
   if (tokens <= 0) return 0;
-  DISPATCH(dtype,
-           hipLaunchKernelGGL(moe_finish_kernel<bf16_t>, dim3(tokens), dim3(256), 0, st, residual, (const bf16_t*)y, weights, pos, topk, (const bf16_t*)shared, gate, n, overwrite),
-           hipLaunchKernelGGL(moe_finish_kernel<float>, dim3(tokens), dim3(256), 0, st, residual, (const float*)y, weights, pos, topk, (const float*)shared, gate, n, overwrite));
+  const bool vec = n % 8 == 0 && (((uintptr_t)residual | (uintptr_t)y | (uintptr_t)shared) & 15) == 0;
+  // launches of a few tokens spread their channels over the grid
+  const int cols = tokens <= 128 ? (n + (vec ? 2047 : 255)) / (vec ? 2048 : 256) : 1;
+#define MF(T, V)                                                                                                   \
+  moe_finish_kernel<T, V><<<dim3(tokens, cols > 64 ? 64 : cols), 256, 0, st>>>(residual, (const T*)y, weights, pos, topk, \
+                                                                               (const T*)shared, gate, n, overwrite)
+  DISPATCH(dtype, if (vec) MF(bf16_t, true); else MF(bf16_t, false), if (vec) MF(float, true); else MF(float, false));
+#undef MF
   return 0;
 }

@@ -51,48 +51,86 @@ __global__ __launch_bounds__(256) void moe_topk_softmax_kernel(const uint16_t* _
 }
 
 // Single-workgroup counting sort.  offsets has n_experts + 1 entries; pos[i] is the sorted
-// row of pair i = t*topk + k; sorted_tok[row] = token of that row, sorted_w[row] (optional) its pair's weight.  Pairs of one expert keep
-// their token order (stable), so results do not depend on scheduling.
+// row of pair i = t*topk + k; sorted_tok[row] = token of that row, sorted_w[row] (optional) its pair's weight.  Pairs of
+// one expert keep their token order (stable), so results do not depend on scheduling.
+// Each of the 16 waves owns a contiguous run of pairs: it counts its run's pairs per expert, the counts turn into the
+// run's first row per expert (expert by expert, run by run), and the wave walks its run 64 pairs at a time, a pair's
+// rank among the 64 being its place among the lanes with the same expert (one ballot per bit of the expert's number).
+#define ALIGN_WAVES 16
 __global__ __launch_bounds__(1024) void moe_align_kernel(const int* __restrict__ ids,
                                                          int* __restrict__ offsets,
                                                          int* __restrict__ pos,
                                                          int* __restrict__ sorted_tok,
                                                          const float* __restrict__ weights,
                                                          float* __restrict__ sorted_w, int n_pairs,
-                                                         int n_experts, int topk) {
-  __shared__ int cnt[ALIGN_MAX_EXPERTS + 1];
-  __shared__ int base[ALIGN_MAX_EXPERTS + 1];
-  const int tid = threadIdx.x;
-  for (int e = tid; e <= n_experts; e += 1024) cnt[e] = 0;
+                                                         int n_experts, int topk, int id_bits) {
+  extern __shared__ int cnt[];  // [ALIGN_WAVES][n_experts]: counts, then next free rows; [n_experts]: totals
+  int* const total = cnt + ALIGN_WAVES * n_experts;
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
+  for (int e = tid; e < ALIGN_WAVES * n_experts; e += 1024) cnt[e] = 0;
   __syncthreads();
-  for (int i = tid; i < n_pairs; i += 1024) atomicAdd(&cnt[ids[i]], 1);
-  __syncthreads();
-  if (tid == 0) {
-    int run = 0;
-    for (int e = 0; e < n_experts; ++e) {
-      base[e] = run;
-      offsets[e] = run;
-      run += cnt[e];
-    }
-    offsets[n_experts] = run;
+  const int run = ((n_pairs + ALIGN_WAVES - 1) / ALIGN_WAVES + 63) & ~63;
+  const int i_lo = wave * run, i_hi = min(n_pairs, i_lo + run);
+  int* const mine = cnt + wave * n_experts;
+  for (int i = i_lo + lane; i < i_hi; i += 64) {
+    const int e = ids[i];
+    if (e >= 0 && e < n_experts) atomicAdd(&mine[e], 1);
   }
   __syncthreads();
-  // stable placement: expert e is handled by wave (e % 16); the wave walks the pair list in
-  // order and ranks its matches with a ballot prefix count
-  const int wave = tid >> 6, lane = tid & 63;
-  for (int e = wave; e < n_experts; e += 16) {
-    int run = base[e];
-    for (int i0 = 0; i0 < n_pairs; i0 += 64) {
-      const int i = i0 + lane;
-      const bool hit = i < n_pairs && ids[i] == e;
-      const unsigned long long m = __ballot(hit);
-      if (hit) {
-        const int rank = __popcll(m & ((1ull << lane) - 1ull));
-        pos[i] = run + rank;
-        sorted_tok[run + rank] = i / topk;
-        if (sorted_w) sorted_w[run + rank] = weights[i];
+  for (int e = tid; e < n_experts; e += 1024) {
+    int sum = 0;
+    for (int w = 0; w < ALIGN_WAVES; ++w) sum += cnt[w * n_experts + e];
+    total[e] = sum;
+  }
+  __syncthreads();
+  if (wave == 0) {  // exclusive prefix over the experts, 64 at a time
+    int base = 0;
+    for (int e0 = 0; e0 < n_experts; e0 += 64) {
+      const int e = e0 + lane;
+      const int v = e < n_experts ? total[e] : 0;
+      int incl = v;
+#pragma unroll
+      for (int off = 1; off < 64; off <<= 1) {
+        const int o = __shfl_up(incl, off, 64);
+        if (lane >= off) incl += o;
       }
-      run += __popcll(m);
+      if (e < n_experts) {
+        total[e] = base + incl - v;
+        offsets[e] = base + incl - v;
+      }
+      base += __shfl(incl, 63, 64);
+    }
+    if (lane == 0) offsets[n_experts] = base;
+  }
+  __syncthreads();
+  for (int e = tid; e < n_experts; e += 1024) {
+    int at = total[e];
+    for (int w = 0; w < ALIGN_WAVES; ++w) {
+      const int c = cnt[w * n_experts + e];
+      cnt[w * n_experts + e] = at;
+      at += c;
+    }
+  }
+  __syncthreads();
+  for (int i0 = i_lo; i0 < i_hi; i0 += 64) {
+    const int i = i0 + lane;
+    const int e = i < i_hi ? ids[i] : -1;
+    const bool ok = e >= 0 && e < n_experts;
+    unsigned long long same = __ballot(ok);
+    for (int b = 0; b < id_bits; ++b) {
+      const unsigned long long set = __ballot(ok && ((e >> b) & 1));
+      same &= ((e >> b) & 1) ? set : ~set;
+    }
+    if (ok) {
+      const unsigned long long below = same & ((1ull << lane) - 1ull);
+      const int row = mine[e] + __popcll(below);
+      pos[i] = row;
+      sorted_tok[row] = i / topk;
+      if (sorted_w) sorted_w[row] = weights[i];
+      // the wave runs in lockstep: every lane has read mine[e] before the last lane of its expert moves it on
+      __builtin_amdgcn_wave_barrier();
+      if ((same >> lane) == 1ull) mine[e] = row + 1;
+      __builtin_amdgcn_wave_barrier();
     }
   }
 }
@@ -143,9 +181,19 @@ VPSA_EXPORT int vpsa_moe_topk_softmax(const void* logits, float* weights, int* i
 
 VPSA_EXPORT int vpsa_moe_align(const int* ids, int* offsets, int* pos, int* sorted_tok,
                                const float* weights, float* sorted_w, int n_pairs, int n_experts, int topk, hipStream_t stream) {
-  if (n_experts > ALIGN_MAX_EXPERTS || (sorted_w && !weights)) return -1;
-  hipLaunchKernelGGL(moe_align_kernel, dim3(1), dim3(1024), 0, stream, ids, offsets, pos,
-                     sorted_tok, weights, sorted_w, n_pairs, n_experts, topk);
+  if (n_experts < 1 || n_experts > ALIGN_MAX_EXPERTS || (sorted_w && !weights)) return -1;
+  const size_t lds = (size_t)(ALIGN_WAVES + 1) * n_experts * sizeof(int);  // 68 KiB at the most
+  static bool attr_set = false;
+  if (lds > 48 * 1024 && !attr_set) {
+    if (hipFuncSetAttribute((const void*)moe_align_kernel, hipFuncAttributeMaxDynamicSharedMemorySize,
+                            (ALIGN_WAVES + 1) * ALIGN_MAX_EXPERTS * (int)sizeof(int)) != hipSuccess)
+      return -2;
+    attr_set = true;
+  }
+  int id_bits = 0;
+  while ((1 << id_bits) < n_experts) ++id_bits;
+  hipLaunchKernelGGL(moe_align_kernel, dim3(1), dim3(1024), lds, stream, ids, offsets, pos,
+                     sorted_tok, weights, sorted_w, n_pairs, n_experts, topk, id_bits);
   return 0;
 }
 

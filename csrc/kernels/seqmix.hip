@@ -1211,15 +1211,23 @@ __device__ __forceinline__ void gru_st2(T* p, int c, int n, float a, float b) {
     if (c + 1 < n) Cv<T>::st(p + c + 1, b);
   }
 }
+// bf16 activations: the hardware's exp2 and reciprocal (about 1e-6 relative at |x| = 10), 32-bit ones: libm and a
+// true division
+template <typename T>
+__device__ __forceinline__ float gru_sigm(float x) {
+  if constexpr (sizeof(T) == 2) return __builtin_amdgcn_rcpf(1.f + __expf(-x));
+  else return sigm(x);
+}
+template <typename T>
 __device__ __forceinline__ void gru_gates(float pz, float px, float& a, float& b) {
-  const float z = sigm(pz);
+  const float z = gru_sigm<T>(pz);
   a = 1.f - z;
-  b = z * (px >= 0.f ? px + 0.5f : sigm(px));
+  b = z * (px >= 0.f ? px + 0.5f : gru_sigm<T>(px));
 }
 
 // PHASE 0: blockIdx.x is a sequence, walked block by block; 1 / 2: blockIdx.x is a piece
 template <typename T, bool VEC, int PHASE>
-__global__ __launch_bounds__(512) void mingru_kernel(
+__global__ __launch_bounds__(512, 4) void mingru_kernel(
     const T* __restrict__ pz, const T* __restrict__ px, const T* __restrict__ pg, long stride, int width,
     const float* __restrict__ bz, const float* __restrict__ bx, float* __restrict__ state, long state_stride,
     const int* __restrict__ seq_cu, const int* __restrict__ seq_state, const int* __restrict__ positions,
@@ -1289,15 +1297,19 @@ __global__ __launch_bounds__(512) void mingru_kernel(
     const int w0 = r0 + GRU_ROWS * wave;
     const int cnt = min(GRU_ROWS, rows - w0);  // rows of this wave (may be <= 0)
     const long at = (long)(row0 + w0) * stride;
-    float a[GRU_ROWS][2], b[GRU_ROWS][2], g[GRU_ROWS][2];
+    float a[GRU_ROWS][2], b[GRU_ROWS][2];
+    constexpr bool RAW = VEC && sizeof(T) == 2;   // gates' inputs wait as pairs of 16 bits: two workgroups per CU
+    uint32_t graw[RAW ? GRU_ROWS : 1];
+    float g[RAW ? 1 : GRU_ROWS][2];
 #pragma unroll
     for (int i = 0; i < GRU_ROWS; ++i) {
 #pragma unroll
-      for (int e = 0; e < 2; ++e) a[i][e] = b[i][e] = g[i][e] = 0.f;
+      for (int e = 0; e < 2; ++e) a[i][e] = b[i][e] = 0.f;
       if (i < cnt) {
         gru_ld2<VEC>(pz + at + i * stride, c, width, a[i]);
         gru_ld2<VEC>(px + at + i * stride, c, width, b[i]);
-        if (PHASE != 1) gru_ld2<VEC>(pg + at + i * stride, c, width, g[i]);
+        if constexpr (PHASE != 1 && RAW) graw[i] = c < width ? *reinterpret_cast<const uint32_t*>(pg + at + i * stride + c) : 0u;
+        else if constexpr (PHASE != 1) gru_ld2<VEC>(pg + at + i * stride, c, width, g[i]);
       }
     }
     float ca[2] = {1.f, 1.f}, cb[2] = {0.f, 0.f};
@@ -1306,7 +1318,7 @@ __global__ __launch_bounds__(512) void mingru_kernel(
       if (i < cnt) {
 #pragma unroll
         for (int e = 0; e < 2; ++e) {
-          gru_gates(a[i][e] + vz[e], b[i][e] + vx[e], a[i][e], b[i][e]);
+          gru_gates<T>(a[i][e] + vz[e], b[i][e] + vx[e], a[i][e], b[i][e]);
           cb[e] = a[i][e] * cb[e] + b[i][e];
           ca[e] *= a[i][e];
         }
@@ -1343,11 +1355,13 @@ __global__ __launch_bounds__(512) void mingru_kernel(
 #pragma unroll
     for (int i = 0; i < GRU_ROWS; ++i)
       if (i < cnt) {
-        float o[2];
+        float o[2], gv[2];
+        if constexpr (RAW) gv[0] = bf16lo(graw[i]), gv[1] = bf16hi(graw[i]);
+        else gv[0] = g[i][0], gv[1] = g[i][1];
 #pragma unroll
         for (int e = 0; e < 2; ++e) {
           mine[e] = a[i][e] * mine[e] + b[i][e];
-          o[e] = mine[e] * g[i][e] * sigm(g[i][e]);
+          o[e] = mine[e] * gv[e] * gru_sigm<T>(gv[e]);
         }
         gru_st2<VEC>(y + (long)(row0 + w0 + i) * width, c, width, o[0], o[1]);
       }
@@ -1382,10 +1396,10 @@ __global__ __launch_bounds__(256) void mingru_step_kernel(
     o[e] = 0.f;
     if (c + e < width) {
       float a, b;
-      gru_gates(z[e] + bz[c + e], x[e] + bx[c + e], a, b);
+      gru_gates<T>(z[e] + bz[c + e], x[e] + bx[c + e], a, b);
       const float s = fresh ? b : a * st[c + e] + b;
       if (slot >= 0) st[c + e] = s;
-      o[e] = s * g[e] * sigm(g[e]);
+      o[e] = s * g[e] * gru_sigm<T>(g[e]);
     }
   }
   gru_st2<VEC>(y + row * width, c, width, o[0], o[1]);

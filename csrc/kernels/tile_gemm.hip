@@ -293,6 +293,16 @@ __global__ __launch_bounds__(512, 2) void tile_gemm_kernel(
 
   // ---- epilogue.  Accumulator [mh][nh][mi][ni]: lane -> output row 128 wr + 64 mh + 16 mi + lane % 16,
   // register e -> column 64 wc + 32 nh + 8 (lane / 16) + 4 ni + e.
+  float rs[2][4];  // the rows' factors, all loads in flight
+  if (EPI == TG_EPI_GLU_CLAMP) {
+#pragma unroll
+    for (int mh = 0; mh < 2; ++mh)
+#pragma unroll
+      for (int mi = 0; mi < 4; ++mi) {
+        const int row = row0 + 128 * wr + 64 * mh + 16 * mi + fr;
+        rs[mh][mi] = row_scale ? row_scale[row < row_end ? row : row_end - 1] : 1.f;
+      }
+  }
 #pragma unroll
   for (int mh = 0; mh < 2; ++mh) {
 #pragma unroll
@@ -301,15 +311,14 @@ __global__ __launch_bounds__(512, 2) void tile_gemm_kernel(
       if (TG_PAIRED(EPI)) {
         const int col = n_idx * 128 + wc * 32 + 8 * fq;
         float v[8];
-        const float rs = (EPI == TG_EPI_GLU_CLAMP && row_scale && row < row_end) ? row_scale[row] : 1.f;
 #pragma unroll
         for (int ni = 0; ni < 2; ++ni)
 #pragma unroll
           for (int e = 0; e < 4; ++e) {
             float gt = acc[mh][0][mi][ni][e], up = acc[mh][1][mi][ni][e];
             if (EPI == TG_EPI_GLU_CLAMP) {
-              gt = fminf(gt * rs, act_limit);
-              up = fminf(fmaxf(up * rs, -act_limit), act_limit) + act_bias;
+              gt = fminf(gt * rs[mh][mi], act_limit);
+              up = fminf(fmaxf(up * rs[mh][mi], -act_limit), act_limit) + act_bias;
               v[4 * ni + e] = gt / (1.f + __expf(-act_alpha * gt)) * up;
             } else if (EPI == TG_EPI_GELU_GLU) {
               // 0.5 g (1 + tanh(y)) = g / (1 + exp(-2 y)),  y = sqrt(2 / pi) (g + 0.044715 g^3)

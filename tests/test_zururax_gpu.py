@@ -215,7 +215,7 @@ def test_expanded_prefill_in_the_engine():
     """Prefill parts large enough to expand keys and values per head for the step (bf16): whole prompts, a
     second large portion over a cached first one, large portions beside decoding requests; the small portions
     and the decoded tokens of the same requests stay in latent space and must agree with them."""
-    from vllm_production_stack_amd.models import zururax
+    from vllm_production_stack_amd.models import latent_mixer
 
     cfg = zo.config_d()
     w = zo.make_weights(cfg, seed=6)
@@ -238,7 +238,7 @@ def test_expanded_prefill_in_the_engine():
                           ["a", "b", "c", "d"]).cpu()
     zo.check_rows(out[2:502], want[:500], 6e-2, "large portion in a mixed batch")
     zo.check_rows(torch.stack([out[0], out[1], out[502]]), torch.stack([la[89], lb[39], lb[6]]), 1e-1, "its neighbours")
-    assert zururax.EXPAND_MIN_ROWS == 256
+    assert latent_mixer.EXPAND_MIN_ROWS == 256
     eng.shutdown()
 
 

@@ -140,7 +140,7 @@ class LatentAttention:
                 o_lat = ops.latent_attention(q_lat, q[:nd, :, m.dim:], pool, lw.cache_offset, meta.dec_block_tables, None,
                                              meta.positions[:nd], lw.sink, m.scale,
                                              splits=getattr(meta, "dec_num_splits", 1) or 1)
-                o[:nd] = torch.bmm(o_lat.transpose(0, 1), lw.w_uv).transpose(0, 1)
+                torch.bmm(o_lat.transpose(0, 1), lw.w_uv, out=o[:nd].transpose(0, 1))
             return o
         # [heads, T, dim] x [heads, dim, kv_rank]: the unrotated query in latent space
         q_lat = torch.bmm(q[:, :, :m.dim].transpose(0, 1), lw.w_uk).transpose(0, 1)
@@ -154,5 +154,7 @@ class LatentAttention:
             ops.latent_attention(q_lat[nd:], q_rot[nd:], pool, lw.cache_offset, meta.pre_block_tables,
                                  meta.pre_row_seq, meta.positions[nd:], lw.sink, m.scale, out=o_lat[nd:],
                                  tiles=(meta.pre_lat_tiles or {}).get(m.heads))
-        # [heads, T, kv_rank] x [heads, kv_rank, vdim] -> [T, heads, vdim]
-        return torch.bmm(o_lat.transpose(0, 1), lw.w_uv).transpose(0, 1).contiguous()
+        # [heads, T, kv_rank] x [heads, kv_rank, vdim], stored as [T, heads, vdim]
+        o = torch.empty((t, m.heads, m.vdim), dtype=q.dtype, device=q.device)
+        torch.bmm(o_lat.transpose(0, 1), lw.w_uv, out=o.transpose(0, 1))
+        return o

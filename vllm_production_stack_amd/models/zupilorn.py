@@ -211,9 +211,8 @@ class ZupilornModel(LatentAttention):
         nq = m.heads * (m.dim + m.rot_dim)
         proj = ops.linear(h, lw.w_in)  # q | KV latent | shared key part
         q = proj[:, :nq].view(t, m.heads, m.dim + m.rot_dim)
-        ops.rope_pairs(q, meta.positions, lw.cos_sin, m.dim, m.rope_dims)
         ops.latent_kv_write(proj[:, nq:nq + m.entry], lw.dkv_norm, meta.positions, meta.slots, lw.cos_sin, pool,
-                            lw.cache_offset, m.kv_rank, m.rot_dim, m.rope_dims, self.cfg.norm_eps)
+                            lw.cache_offset, m.kv_rank, m.rot_dim, m.rope_dims, self.cfg.norm_eps, q=q, q_col=m.dim)
         o = self.latent_heads(lw, q, pool, meta)
         return ops.linear(o.view(t, m.heads * m.vdim), lw.w_o)
 

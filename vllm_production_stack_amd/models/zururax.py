@@ -158,11 +158,12 @@ class ZururaxModel(LatentAttention):
         col = m.q_rank
         cq = ops.rms_norm_rows(proj[:, :col], lw.dq_norm, eps)
         q = ops.linear(cq, lw.w_uq).view(t, m.heads, m.dim + m.rot_dim)
-        ops.rope_pairs(q, meta.positions, lw.cos_sin, m.dim, m.rope_dims)
         if m.kv_from is None:
             ops.latent_kv_write(proj[:, col:col + m.entry], lw.dkv_norm, meta.positions, meta.slots, lw.cos_sin, pool,
-                                lw.cache_offset, m.kv_rank, m.rot_dim, m.rope_dims, eps)
+                                lw.cache_offset, m.kv_rank, m.rot_dim, m.rope_dims, eps, q=q, q_col=m.dim)
             col += m.entry
+        else:
+            ops.rope_pairs(q, meta.positions, lw.cos_sin, m.dim, m.rope_dims)
         o = self.latent_heads(lw, q, pool, meta)
         if m.out_gate:
             ops.sigmoid_gate(o, proj[:, col:col + m.heads])

@@ -196,19 +196,26 @@ def _layer_base(pool, offset: int, entry: int):
 
 
 def latent_kv_write(x, weight, positions, slots, cos_sin, pool, offset: int, rank: int, rot: int, rot_dims: int,
-                    eps: float):
-    """Rows of x [T, rank + rot] (a view) -> cache entries: RMS-normed latent | rotated key part."""
+                    eps: float, q=None, q_col: int = 0):
+    """Rows of x [T, rank + rot] (a view) -> cache entries: RMS-normed latent | rotated key part.  ``q`` [T, heads, d] (a
+    view): its columns [q_col, q_col + rot_dims) of every head turn as well, in place (``rope_pairs`` in the same launch)."""
     if not x.is_cuda:
+        if q is not None:
+            reference.rope_pairs(q, positions, cos_sin, q_col, rot_dims)
         return reference.latent_kv_write(x, weight, positions, slots, cos_sin, pool, offset, rank, rot, rot_dims, eps)
     o = _ops()
     _f32(weight, cos_sin)
     assert _rows(x) and x.shape[1] == rank + rot and positions.dtype == torch.int32 and slots.dtype == torch.int64
-    assert cos_sin.shape[1] == rot_dims and weight.numel() == rank
+    assert cos_sin.shape[1] == rot_dims and weight.numel() == rank and rot_dims <= rot
+    assert q is None or (q.dim() == 3 and q.stride(2) == 1 and q.shape[0] == x.shape[0] and q_col + rot_dims <= q.shape[2])
     o._check(o._kernels().vpsa_latent_kv_write(o._p(x), c_long(x.stride(0)), o._p(weight), o._p(positions), o._p(slots),
                                                o._p(cos_sin), _layer_base(pool, offset, rank + rot),
                                                c_long(pool.stride(0)), c_int(x.shape[0]), c_int(rank), c_int(rot),
-                                               c_int(rot_dims), c_float(eps), c_int(_dt(x, pool)), o._stream()),
-             "latent_kv_write")
+                                               c_int(rot_dims), c_float(eps), o._p(q),
+                                               c_long(q.stride(0) if q is not None else 0),
+                                               c_long(q.stride(1) if q is not None else 0),
+                                               c_int(q.shape[1] if q is not None else 0), c_int(q_col),
+                                               c_int(_dt(x, pool, q)), o._stream()), "latent_kv_write")
 
 
 def rope_pairs(q, positions, cos_sin, col0: int, rot_dims: int):
