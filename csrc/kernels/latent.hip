@@ -10,8 +10,8 @@
 //   latent_kv_write    a token's compressed KV entry: RMS-normed latent | rotated shared key part
 //                      -> paged cache row [rank + rot]; optionally the rotation of the query heads as well
 //   rope_pairs         interleaved-pair rotary embedding of a column range of every head, in place
-//   latent_attention   causal attention of query rows in latent space over the paged entries with an
-//                      optional per-head sink logit in the softmax denominator
+//   latent_attention   causal attention of query rows in latent space over the paged entries, whole or within a
+//                      sliding window, with an optional per-head sink logit in the softmax denominator
 //   sigmoid_gate       y[t, h, :] *= sigmoid(g[t, h])
 //   relu_sq            y = relu(x)^2
 //   glu_clamp          y = g' * sigmoid(alpha g') * (u' + bias),  g' = min(g, limit), u' = clamp(u, +-limit)
@@ -256,7 +256,7 @@ __global__ __launch_bounds__(256) void rope_pairs_kernel(T* __restrict__ q, long
 // Latent attention, plain form.  One 256-thread workgroup per (query row, head).  The query is
 // q_lat [rank] (the head's unrotated query carried into latent space) | q_rot [rot]; key j of the
 // row's sequence is the cache entry [rank + rot] and its value the entry's first rank columns.
-//   score_j = (q_lat . c_j + q_rot . r_j) * scale,   j <= position
+//   score_j = (q_lat . c_j + q_rot . r_j) * scale,   position - window < j <= position
 //   out     = sum_j exp(score_j - m) c_j / (sum_j exp(score_j - m) + exp(sink - m))
 // Keys are taken 256 at a time (a thread scores one key, then owns output columns tid, tid+256, ..).
 // ---------------------------------------------------------------------------------
@@ -267,7 +267,7 @@ __global__ __launch_bounds__(256) void latent_attention_kernel(
     const T* __restrict__ q_lat, long ql_row, long ql_head, const T* __restrict__ q_rot, long qr_row, long qr_head,
     const T* __restrict__ cache, long page_stride, const int* __restrict__ block_tables, int bt_stride,
     const int* __restrict__ row_seq, const int* __restrict__ positions, const float* __restrict__ sink,
-    T* __restrict__ out, long o_row, long o_head, int rank, int rot, float scale) {
+    T* __restrict__ out, long o_row, long o_head, int rank, int rot, float scale, int window) {
   extern __shared__ float smem[];
   float* qs = smem;             // [rank + rot], pre-scaled
   float* ps = smem + rank + rot;  // [256]
@@ -275,6 +275,7 @@ __global__ __launch_bounds__(256) void latent_attention_kernel(
   const int row = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
   const int width = rank + rot;
   const int ctx = positions[row] + 1;
+  const int lo = max(0, ctx - window);  // the first key seen; a step of 256 keys always holds one that is
   const int seq = row_seq ? row_seq[row] : row;
   const int* bt = block_tables + (long)seq * bt_stride;
   for (int i = tid; i < rank; i += 256) qs[i] = Conv<T>::ld(q_lat + row * ql_row + h * ql_head + i) * scale;
@@ -285,7 +286,7 @@ __global__ __launch_bounds__(256) void latent_attention_kernel(
 #pragma unroll
   for (int c = 0; c < LAT_MAX_COLS; ++c) acc[c] = 0.f;
   __syncthreads();
-  for (int j0 = 0; j0 < ctx; j0 += 256) {
+  for (int j0 = lo; j0 < ctx; j0 += 256) {
     const int j = j0 + tid;
     float s = -INFINITY;
     if (j < ctx) {
@@ -434,12 +435,14 @@ __global__ __launch_bounds__(64) void group_topk_kernel(const float* __restrict_
 // c = s + bias, weighted by s.  Experts form `groups` equal runs of neighbours, a group scores its largest c and
 // only the `keep` best groups take part (the rest count as minus infinity; c may be negative).  The last
 // n - experts outputs are identity experts: a chosen one adds its score to gate[t] and leaves the pair list
-// (weight 0, id = park).  Ties go to the lower index.  One wave per token.
+// (weight 0, id = park).  normalize: the chosen scores are divided by their sum, which makes them the softmax over
+// the chosen logits alone.  Ties go to the lower index.  One wave per token.
 __global__ __launch_bounds__(64) void route_softmax_kernel(const float* __restrict__ logits, int cols,
                                                            const float* __restrict__ bias,
                                                            float* __restrict__ weights, int* __restrict__ ids,
                                                            float* __restrict__ gate, int n, int experts, int groups,
-                                                           int keep, int topk, float route_scale, int park) {
+                                                           int keep, int topk, float route_scale, int park,
+                                                           int normalize) {
   __shared__ float s[ROUTE_MAX_EXPERTS];
   __shared__ float c[ROUTE_MAX_EXPERTS];
   __shared__ float gs[ROUTE_MAX_EXPERTS];
@@ -478,7 +481,7 @@ __global__ __launch_bounds__(64) void route_softmax_kernel(const float* __restri
       for (int e = g * per; e < (g + 1) * per; ++e) c[e] = -INFINITY;
   }
   __syncthreads();
-  float gsum = 0.f;
+  float gsum = 0.f, wsum = 0.f;
   for (int k = 0; k < topk; ++k) {
     float best = -INFINITY;
     int bi = 0x7fffffff;
@@ -494,6 +497,7 @@ __global__ __launch_bounds__(64) void route_softmax_kernel(const float* __restri
       const bool ident = !none && bi >= experts;
       const float w = none ? 0.f : s[bi] * route_scale;
       if (ident) gsum += w;
+      wsum += w;
       weights[t * topk + k] = (ident || none) ? 0.f : w;
       ids[t * topk + k] = (ident || none) ? park : bi;
     }
@@ -501,6 +505,8 @@ __global__ __launch_bounds__(64) void route_softmax_kernel(const float* __restri
     if (lane == 0 && !none) c[bi] = -INFINITY;
     __syncthreads();
   }
+  if (lane == 0 && normalize)
+    for (int k = 0; k < topk; ++k) weights[t * topk + k] *= route_scale / wsum;
   if (lane == 0 && gate) gate[t] = gsum;
 }
 
@@ -1024,15 +1030,16 @@ VPSA_EXPORT int vpsa_latent_attention(const void* q_lat, long ql_row, long ql_he
                                       long qr_head, const void* cache, long page_stride, const int* block_tables,
                                       int bt_stride, const int* row_seq, const int* positions, const float* sink,
                                       void* out, long o_row, long o_head, int rows, int heads, int rank, int rot,
-                                      float scale, int dtype, hipStream_t st) {
+                                      float scale, int window, int dtype, hipStream_t st) {
   if (rows <= 0) return 0;
+  if (window < 1) return -1;
   if (rank > LAT_MAX_COLS * 256 || heads > 65535) return -1;
   const size_t lds = (size_t)(rank + rot + 256) * sizeof(float);
   if (lds > 60 * 1024) return -1;
   dim3 grid(rows, heads);
   DISPATCH(dtype,
-           hipLaunchKernelGGL(latent_attention_kernel<bf16_t>, grid, dim3(256), lds, st, (const bf16_t*)q_lat, ql_row, ql_head, (const bf16_t*)q_rot, qr_row, qr_head, (const bf16_t*)cache, page_stride, block_tables, bt_stride, row_seq, positions, sink, (bf16_t*)out, o_row, o_head, rank, rot, scale),
-           hipLaunchKernelGGL(latent_attention_kernel<float>, grid, dim3(256), lds, st, (const float*)q_lat, ql_row, ql_head, (const float*)q_rot, qr_row, qr_head, (const float*)cache, page_stride, block_tables, bt_stride, row_seq, positions, sink, (float*)out, o_row, o_head, rank, rot, scale));
+           hipLaunchKernelGGL(latent_attention_kernel<bf16_t>, grid, dim3(256), lds, st, (const bf16_t*)q_lat, ql_row, ql_head, (const bf16_t*)q_rot, qr_row, qr_head, (const bf16_t*)cache, page_stride, block_tables, bt_stride, row_seq, positions, sink, (bf16_t*)out, o_row, o_head, rank, rot, scale, window),
+           hipLaunchKernelGGL(latent_attention_kernel<float>, grid, dim3(256), lds, st, (const float*)q_lat, ql_row, ql_head, (const float*)q_rot, qr_row, qr_head, (const float*)cache, page_stride, block_tables, bt_stride, row_seq, positions, sink, (float*)out, o_row, o_head, rank, rot, scale, window));
   return 0;
 }
 
@@ -1161,13 +1168,13 @@ VPSA_EXPORT int vpsa_soft_cap(const void* x, void* y, long n, float cap, int dty
 // into a bucket no product visits, 0 for callers that run every pair.
 VPSA_EXPORT int vpsa_route_softmax(const float* logits, int cols, const float* bias, float* weights, int* ids,
                                    float* gate, int tokens, int n, int experts, int groups, int keep, int topk,
-                                   float route_scale, int park, hipStream_t st) {
+                                   float route_scale, int park, int normalize, hipStream_t st) {
   if (tokens <= 0) return 0;
   if (n > ROUTE_MAX_EXPERTS || experts > n || groups < 1 || n % groups || keep < 1 || keep > groups || cols < n ||
-      topk < 1 || (experts < n && !gate))
+      topk < 1 || (experts < n && !gate) || (normalize && experts < n))
     return -1;
   hipLaunchKernelGGL(route_softmax_kernel, dim3(tokens), dim3(64), 0, st, logits, cols, bias, weights, ids, gate, n,
-                     experts, groups, keep, topk, route_scale, park);
+                     experts, groups, keep, topk, route_scale, park, normalize);
   return 0;
 }
 

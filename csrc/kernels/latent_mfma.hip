@@ -19,6 +19,10 @@
 // are XOR-swizzled with (row / 8) % 8: the transposing stores of neighbouring lanes lie 8 rows apart.)
 // The next page's global loads are issued before the current page is multiplied.
 //
+// With a sliding window of `window` positions (a query at position p sees keys p - window + 1 .. p) the walk starts
+// at the page of the first key that the tile's earliest query sees; only pages that hold a key some slot does not
+// see are masked key by key.
+//
 // Softmax state (running max, sum) is fp32 per slot; an optional per-head sink logit starts the state
 // (max = sink, sum = 1).  With key-range splits every split writes unnormalised partial outputs and
 // (max, sum) to a workspace and a merge kernel adds the sink and normalises.
@@ -37,8 +41,8 @@ __global__ __launch_bounds__(256) void latent_mfma_kernel(
     const uint16_t* __restrict__ q_lat, long ql_row, long ql_head, const uint16_t* __restrict__ q_rot, long qr_row,
     long qr_head, const uint16_t* __restrict__ cache, long page_stride, const int* __restrict__ block_tables,
     int bt_stride, const int* __restrict__ tiles, const int* __restrict__ positions, int heads,
-    const float* __restrict__ sink, uint16_t* __restrict__ out, long o_row, long o_head, float scale, int splits,
-    float* __restrict__ ws_o, float* __restrict__ ws_ml) {
+    const float* __restrict__ sink, uint16_t* __restrict__ out, long o_row, long o_head, float scale, int window,
+    int splits, float* __restrict__ ws_o, float* __restrict__ ws_ml) {
   constexpr int ENTRY = RANK + ROT;
   constexpr int KS = ENTRY / 32;
   constexpr int DT = RANK / 16;
@@ -71,8 +75,10 @@ __global__ __launch_bounds__(256) void latent_mfma_kernel(
   const long row = t.row0 + tok;
   const int my_pos = valid ? t.pos0 + tok : -1;
   const int n_pages = (t.pos0 + t.n_tok + PAGE - 1) / PAGE;
-  const int per = (n_pages + splits - 1) / splits;
-  const int p_begin = blockIdx.y * per, p_end = min(n_pages, p_begin + per);
+  const int p_first = max(0, t.pos0 - window + 1) / PAGE;
+  const int per = (n_pages - p_first + splits - 1) / splits;
+  const int p_begin = p_first + blockIdx.y * per, p_end = min(n_pages, p_begin + per);
+  const int my_first = my_pos - window;  // keys beyond it, up to my_pos, are seen
   const int* bt = block_tables + (long)t.seq * bt_stride;
 
   bf16x8 qf[KS];
@@ -166,12 +172,14 @@ __global__ __launch_bounds__(256) void latent_mfma_kernel(
         s[nt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, qf[ks], s[nt], 0, 0, 0);
       }
     float mx = -INFINITY;
+    // every slot of the tile sees the whole page: nothing to mask
+    const bool whole = p * PAGE + PAGE - 1 <= t.pos0 && p * PAGE > t.pos0 + t.n_tok - 1 - window;
 #pragma unroll
     for (int nt = 0; nt < 4; ++nt)
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
         const int key = p * PAGE + 16 * nt + 4 * g + e;
-        const float v = key <= my_pos ? s[nt][e] * scale : -INFINITY;
+        const float v = whole || (key <= my_pos && key > my_first) ? s[nt][e] * scale : -INFINITY;
         s[nt][e] = v;
         mx = fmaxf(mx, v);
       }
@@ -278,7 +286,7 @@ template <int RANK, int ROT>
 int launch(const void* q_lat, long ql_row, long ql_head, const void* q_rot, long qr_row, long qr_head,
            const void* cache, long page_stride, const int* block_tables, int bt_stride, const int* tiles,
            const int* positions, int n_tiles, int heads, const float* sink, void* out, long o_row, long o_head,
-           float scale, int splits, float* ws_o, float* ws_ml, hipStream_t st) {
+           float scale, int window, int splits, float* ws_o, float* ws_ml, hipStream_t st) {
   constexpr int LDS = 64 * ((RANK + ROT) * 2 + 16) + RANK * (64 * 2 + 16);
   static bool attr_set = false;
   if (!attr_set) {
@@ -290,7 +298,7 @@ int launch(const void* q_lat, long ql_row, long ql_head, const void* q_rot, long
   latent_mfma_kernel<RANK, ROT><<<dim3(n_tiles, splits), dim3(256), LDS, st>>>(
       (const uint16_t*)q_lat, ql_row, ql_head, (const uint16_t*)q_rot, qr_row, qr_head, (const uint16_t*)cache,
       page_stride, block_tables, bt_stride, tiles, positions, heads, sink, (uint16_t*)out, o_row, o_head, scale,
-      splits, ws_o, ws_ml);
+      window, splits, ws_o, ws_ml);
   if (splits > 1)
     latent_merge_kernel<<<dim3(n_tiles, 64), dim3(128), 0, st>>>(ws_o, ws_ml, tiles, heads, sink, (uint16_t*)out,
                                                                  o_row, o_head, splits, RANK);
@@ -316,21 +324,24 @@ VPSA_EXPORT int vpsa_latent_mfma_supported(int rank, int rot) {
 // tiles: int32 [n_tiles, 6] = (sequence, first query row, tokens, position of the first token, first head,
 // heads per token) with tokens * heads <= 64 and sequence < 0 for an unused entry; null = decode rows
 // (n_tiles = rows * ceil(heads / 64), positions [rows]).  Row and head strides in elements; every query
-// and output vector 16-byte / 8-byte aligned.  splits > 1 needs ws_o [n_tiles * splits * 64 * rank] and
+// and output vector 16-byte / 8-byte aligned.  window >= 1 (a query sees itself and the window - 1 entries before
+// it; any window of at least the context length is plain causal attention).  splits > 1 needs ws_o [n_tiles * splits * 64 * rank] and
 // ws_ml [n_tiles * splits * 64 * 2] floats.
 VPSA_EXPORT int vpsa_latent_attention_mfma(const void* q_lat, long ql_row, long ql_head, const void* q_rot,
                                            long qr_row, long qr_head, const void* cache, long page_stride,
                                            const int* block_tables, int bt_stride, const int* tiles,
                                            const int* positions, int n_tiles, int heads, const float* sink, void* out,
-                                           long o_row, long o_head, int rank, int rot, float scale, int splits,
-                                           float* ws_o, float* ws_ml, hipStream_t st) {
+                                           long o_row, long o_head, int rank, int rot, float scale, int window,
+                                           int splits, float* ws_o, float* ws_ml, hipStream_t st) {
   if (n_tiles <= 0) return 0;
+  if (window < 1) return -1;
   if (splits < 1 || splits > 65535 || (splits > 1 && (!ws_o || !ws_ml)) || (!tiles && !positions)) return -1;
   if (((ql_row | ql_head | qr_row | qr_head) & 7) || ((o_row | o_head) & 3) || (page_stride & 7)) return -1;
 #define LAT_CASE(R, C)                                                                                              \
   if (rank == R && rot == C)                                                                                        \
     return launch<R, C>(q_lat, ql_row, ql_head, q_rot, qr_row, qr_head, cache, page_stride, block_tables, bt_stride, \
-                        tiles, positions, n_tiles, heads, sink, out, o_row, o_head, scale, splits, ws_o, ws_ml, st);
+                        tiles, positions, n_tiles, heads, sink, out, o_row, o_head, scale, window, splits, ws_o,      \
+                        ws_ml, st);
   LAT_SHAPES(LAT_CASE)
 #undef LAT_CASE
   return -1;

@@ -541,7 +541,6 @@ VPSA_EXPORT int vpsa_moe_mfma_act(const void* x, const void* w13, const void* w2
 VPSA_EXPORT int vpsa_moe_mfma(const void* x, const void* w13, const void* w2, const int* offsets,
                               const int* sorted_tok, void* act, void* y, int tokens, int topk,
                               int n_experts, int hidden, int inter, hipStream_t stream) {
-  if (n_experts > MAX_EXPERTS) return -1;
   return vpsa_moe_mfma_act(x, w13, w2, offsets, sorted_tok, act, y, tokens, topk, n_experts, hidden, inter, 0.f,
                            1.f, 0.f, nullptr, stream);
 }

@@ -16,7 +16,8 @@
 //   window_attention   softmax(cap tanh(q k scale / cap)) with a sink in the denominator over the keys
 //                      j <= i with i - j < window or j < keep_first (or: of i's own chunk of positions; or: of the
 //                      window and one pooled entry per block of tokens before it), applied to the values of EVERY
-//                      KV head or of the head's own
+//                      KV head or of the head's own; optionally times a sigmoid gate per head, in the activation dtype
+//   window_kv_write    keys and values of a projection -> paged cache as they are (the layout window_attention reads)
 //   mix_heads          out[t, h] = sum_g talk[h, g] u[t, g, kv_head(h)]
 //   xielu              z > 0: a_p z^2 + z / 2;  else a_n (exp(z) - 1 - z) + z / 2
 //   qk_norm_write      q and k heads to unit root mean square (a weight per channel, a rotation of the first
@@ -524,6 +525,54 @@ __global__ __launch_bounds__(256) void qk_norm_write_kernel(const T* __restrict_
   }
 }
 
+// Keys and values of the step to the page layout of window_attention as they are (designs without norm or rotation,
+// whose queries the attention reads from the projection itself).  A workgroup takes 64 rows and 64 channels: keys are
+// copied row by row; values are turned through LDS, so that a channel's 64 tokens go out side by side (the rows of a
+// prompt's portion have neighbouring slots).  vec: key rows can be moved 16 bytes at a time.
+constexpr int KVW = 64;
+
+template <typename T>
+__global__ __launch_bounds__(256) void window_kv_write_kernel(const T* __restrict__ k, const T* __restrict__ v,
+                                                              long p_stride, const long* __restrict__ slots,
+                                                              T* __restrict__ cache, long page_stride, int rows, int nk,
+                                                              int nv, int vec) {
+  constexpr int RUN = 16 / sizeof(T);
+  __shared__ long base[KVW];  // where the row's token lies: its page's first element, and its place in the page
+  __shared__ int place[KVW];
+  __shared__ T tile[KVW][KVW + 1];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const long row0 = (long)blockIdx.x * KVW;
+  const int n = min((long)KVW, rows - row0);
+  if (tid < KVW) {
+    const long slot = tid < n ? slots[row0 + tid] : -1;
+    base[tid] = slot < 0 ? -1 : slot / PAGE * page_stride;
+    place[tid] = (int)(slot < 0 ? 0 : slot % PAGE);
+  }
+  __syncthreads();
+  const int k_blocks = (nk + KVW - 1) / KVW;
+  if ((int)blockIdx.y < k_blocks) {
+    const int c0 = blockIdx.y * KVW, nc = min(KVW, nk - c0);
+    const int step = vec ? RUN : 1, per = nc / step;  // (nc is a multiple of RUN with vec)
+    for (int i = tid; i < n * per; i += 256) {
+      const int r = i / per, c = c0 + i % per * step;
+      if (base[r] < 0) continue;
+      const T* src = k + (row0 + r) * p_stride + c;
+      T* dst = cache + base[r] + (long)place[r] * nk + c;
+      if (vec) *reinterpret_cast<u32x4*>(dst) = *reinterpret_cast<const u32x4*>(src);
+      else *dst = *src;
+    }
+    return;
+  }
+  const int c0 = (blockIdx.y - k_blocks) * KVW, nc = min(KVW, nv - c0);
+  for (int r = wave; r < n; r += 4)
+    if (lane < nc) tile[r][lane] = v[(row0 + r) * p_stride + c0 + lane];
+  __syncthreads();
+  if (lane < n && base[lane] >= 0) {
+    T* dst = cache + base[lane] + (long)PAGE * nk + place[lane];
+    for (int c = wave; c < nc; c += 4) dst[(long)(c0 + c) * PAGE] = tile[lane][c];
+  }
+}
+
 // Pooled entries of a windowed attention that also sees a mean key and value per block of `pool` tokens.  A row
 // of the step at position p with (p + 1) % pool == 0 completes block b = p / pool; the
 // block's keys and values are read back from the pages (as the cache holds them, whichever step wrote them), summed
@@ -789,7 +838,8 @@ __device__ __forceinline__ bool key_seen(int j, int p, int window, int keep_firs
 // Plain kernel, every size and both dtypes.  One workgroup per (row, query head), four pages per step: a thread
 // scores one key, then owns value channels and walks the step's keys in runs of 16 bytes.
 // out [rows, heads, kv_heads, vdim] fp32: the head's softmax weights applied to the values of every KV head
-// (the head mixing that follows needs them).
+// (the head mixing that follows needs them).  gate: the head's output times sigmoid(gate[row, head]); out_t: out is
+// in the activation dtype (what an output projection reads).
 constexpr int WA_KEYS = 256;
 constexpr int WA_ACC = 8;  // kv_heads * vdim <= 256 * WA_ACC
 
@@ -797,9 +847,9 @@ template <typename T>
 __global__ __launch_bounds__(256) void window_attention_kernel(
     const T* __restrict__ q, long q_stride, const T* __restrict__ cache, long page_stride,
     const int* __restrict__ block_tables, int bt_stride, const int* __restrict__ row_seq,
-    const int* __restrict__ positions, const float* __restrict__ sink, float* __restrict__ out, int heads, int kv_heads,
+    const int* __restrict__ positions, const float* __restrict__ sink, void* __restrict__ out, int heads, int kv_heads,
     int dim, int vdim, int window, int keep_first, float scale, float softcap, int own, int mode, int pool,
-    long pool_off, int maps) {
+    long pool_off, int maps, const T* __restrict__ gate, long g_stride, int out_t) {
   // own: only the values of the head's own KV head (out [rows, heads, vdim]); designs without head mixing
   // maps: key heads per value head (kv_heads counts key heads; key head g reads the values of head g / maps)
   extern __shared__ float sm[];
@@ -871,11 +921,15 @@ __global__ __launch_bounds__(256) void window_attention_kernel(
     m = mn;
     __syncthreads();
   }
-  const float inv = l > 0.f ? 1.f / l : 0.f;
+  float inv = l > 0.f ? 1.f / l : 0.f;
+  if (gate) inv *= sigm(Cv<T>::ld(gate + row * g_stride + head));
 #pragma unroll
   for (int a = 0; a < WA_ACC; ++a) {
     const int c = a * 256 + tid;
-    if (c < nv) out[(row * heads + head) * (long)nv + c] = acc[a] * inv;
+    const long at = (row * heads + head) * (long)nv + c;
+    if (c >= nv) continue;
+    if (out_t) Cv<T>::st((T*)out + at, acc[a] * inv);
+    else ((float*)out)[at] = acc[a] * inv;
   }
 }
 
@@ -894,9 +948,11 @@ template <int DIM, int VALL, int NSUB>
 __global__ __launch_bounds__(256) void window_mfma_kernel(
     const uint16_t* __restrict__ q, long q_stride, const uint16_t* __restrict__ cache, long page_stride,
     const int* __restrict__ block_tables, int bt_stride, const int* __restrict__ tiles,
-    const int* __restrict__ positions, const float* __restrict__ sink, float* __restrict__ out, int heads, int kv_heads,
+    const int* __restrict__ positions, const float* __restrict__ sink, void* __restrict__ out, int heads, int kv_heads,
     int window, int keep_first, float scale, float softcap, int splits, float* __restrict__ ws_o,
-    float* __restrict__ ws_ml, int n_chunks, int own, int mode, int pool, long pool_off, int maps) {
+    float* __restrict__ ws_ml, int n_chunks, int own, int mode, int pool, long pool_off, int maps,
+    const uint16_t* __restrict__ gate, long g_stride, int out_t) {
+  // gate / out_t: as for the plain kernel
   // mode / pool / pool_off: see PageWalk.  maps (own only): key heads per value head
   // own: a slot's weights meet the values of its own KV head only (n_chunks chunks of VALL channels per KV head,
   // out [rows, heads, n_chunks * VALL]); else those of every KV head (n_chunks chunks over all of them)
@@ -1004,6 +1060,9 @@ __global__ __launch_bounds__(256) void window_mfma_kernel(
     if (!wave_active) continue;
     const int j0 = walk.page(i) * PAGE;
     const bool pooled = walk.pooled(i);
+    // every slot of the tile sees the whole page: nothing to mask
+    const int pos1 = pos0 + n_rows - 1;
+    const bool whole = !pooled && j0 + PAGE - 1 <= pos0 && (mode == 1 ? j0 >= pos1 - pos1 % window : j0 > pos1 - window);
     f32x4 s[NSUB][4];
 #pragma unroll
     for (int u = 0; u < NSUB; ++u)
@@ -1029,7 +1088,7 @@ __global__ __launch_bounds__(256) void window_mfma_kernel(
         for (int e = 0; e < 4; ++e) {
           const int j = j0 + 32 * (nt >> 1) + 8 * g + 4 * (nt & 1) + e;
           float v = -INFINITY;
-          if (pooled ? j < my_blocks[u] : key_seen(j, my_pos[u], window, keep_first, mode)) {
+          if (whole || (pooled ? j < my_blocks[u] : key_seen(j, my_pos[u], window, keep_first, mode))) {
             v = s[u][nt][e] * scale;
             if (softcap > 0.f) {  // cap * tanh(v / cap), tanh(x) = 1 - 2 / (exp(2 x) + 1)
               const float x = v * inv_cap;
@@ -1085,10 +1144,21 @@ __global__ __launch_bounds__(256) void window_mfma_kernel(
   for (int u = 0; u < NSUB; ++u) {
     if (!valid[u]) continue;
     if (splits == 1) {
-      const float inv = l[u] > 0.f ? 1.f / l[u] : 0.f;
-      float* dst = out + (row[u] * heads + head[u]) * vall_total + (long)chunk * VALL + 4 * g;
+      float inv = l[u] > 0.f ? 1.f / l[u] : 0.f;
+      if (gate) inv *= sigm(bf16_bits_to_f32(gate[row[u] * g_stride + head[u]]));
+      const long at = (row[u] * heads + head[u]) * vall_total + (long)chunk * VALL + 4 * g;
+      if (out_t) {
+        uint16_t* dst = (uint16_t*)out + at;
 #pragma unroll
-      for (int dt = 0; dt < DT; ++dt) *reinterpret_cast<f32x4*>(dst + 16 * dt) = o[u][dt] * inv;
+        for (int dt = 0; dt < DT; ++dt) {
+          u32x2 w = {pack_bf16x2(o[u][dt][0] * inv, o[u][dt][1] * inv), pack_bf16x2(o[u][dt][2] * inv, o[u][dt][3] * inv)};
+          *reinterpret_cast<u32x2*>(dst + 16 * dt) = w;
+        }
+      } else {
+        float* dst = (float*)out + at;
+#pragma unroll
+        for (int dt = 0; dt < DT; ++dt) *reinterpret_cast<f32x4*>(dst + 16 * dt) = o[u][dt] * inv;
+      }
     } else {
       const long rec = (row[u] * heads + head[u]) * splits + blockIdx.z;
       float* dst = ws_o + rec * vall_total + (long)chunk * VALL + 4 * g;
@@ -1104,8 +1174,9 @@ __global__ __launch_bounds__(256) void window_mfma_kernel(
 
 // One workgroup per (row, head): out = sum_s o_s exp(m_s - M) / (sum_s l_s exp(m_s - M) + exp(sink - M))
 __global__ __launch_bounds__(128) void window_merge_kernel(const float* __restrict__ ws_o, const float* __restrict__ ws_ml,
-                                                           const float* __restrict__ sink, float* __restrict__ out,
-                                                           int heads, int vall, int splits) {
+                                                           const float* __restrict__ sink, void* __restrict__ out,
+                                                           int heads, int vall, int splits,
+                                                           const uint16_t* __restrict__ gate, long g_stride, int out_t) {
   const long pair = blockIdx.x;
   const int head = (int)(pair % heads);
   float big = sink ? sink[head] : -INFINITY;
@@ -1115,14 +1186,16 @@ __global__ __launch_bounds__(128) void window_merge_kernel(const float* __restri
     const float ms = ws_ml[2 * (pair * splits + s)];
     if (ms != -INFINITY) den += ws_ml[2 * (pair * splits + s) + 1] * __expf(ms - big);
   }
-  const float inv = den > 0.f ? 1.f / den : 0.f;
+  float inv = den > 0.f ? 1.f / den : 0.f;
+  if (gate) inv *= sigm(bf16_bits_to_f32(gate[pair / heads * g_stride + head]));
   for (int c = threadIdx.x; c < vall; c += 128) {
     float acc = 0.f;
     for (int s = 0; s < splits; ++s) {
       const float ms = ws_ml[2 * (pair * splits + s)];
       if (ms != -INFINITY) acc += ws_o[(pair * splits + s) * vall + c] * __expf(ms - big);
     }
-    out[pair * vall + c] = acc * inv;
+    if (out_t) Cv<bf16_t>::st((bf16_t*)out + pair * vall + c, acc * inv);
+    else ((float*)out)[pair * vall + c] = acc * inv;
   }
 }
 
@@ -1597,6 +1670,21 @@ VPSA_EXPORT int vpsa_qk_norm_write(const void* proj, long p_stride, int heads, i
   return 0;
 }
 
+// k / v: the first key and value column of the projection rows (row stride p_stride); nk / nv: key and value channels
+// per token of the layer's page region (all heads); slots < 0: not cached
+VPSA_EXPORT int vpsa_window_kv_write(const void* k, const void* v, long p_stride, const long* slots, void* cache,
+                                     long page_stride, int rows, int nk, int nv, int dt, hipStream_t stream) {
+  if (rows <= 0) return 0;
+  if (nk < 1 || nv < 1) return 2;
+  const int run = dt == 0 ? 8 : 4;
+  const int vec = nk % run == 0 && p_stride % run == 0 && page_stride % run == 0 &&
+                  (((uintptr_t)k | (uintptr_t)cache) & 15) == 0;
+  const dim3 grid((rows + KVW - 1) / KVW, (nk + KVW - 1) / KVW + (nv + KVW - 1) / KVW);
+  SM_DISPATCH(dt, (window_kv_write_kernel<T><<<grid, 256, 0, stream>>>((const T*)k, (const T*)v, p_stride, slots, (T*)cache,
+                                                                       page_stride, rows, nk, nv, vec)));
+  return 0;
+}
+
 // nk / nv: key and value channels per token of the layer's page regions (all heads)
 VPSA_EXPORT int vpsa_pool_blocks(void* cache, long page_stride, long pool_off, const int* block_tables, int bt_stride,
                                  const int* row_seq, const int* positions, const long* slots, int rows, int nk, int nv,
@@ -1640,9 +1728,10 @@ VPSA_EXPORT int vpsa_short_conv_qkv(const void* proj, long p_stride, const float
 
 VPSA_EXPORT int vpsa_window_attention(const void* q, long q_stride, const void* cache, long page_stride,
                                       const int* block_tables, int bt_stride, const int* row_seq, const int* positions,
-                                      const float* sink, float* out, int rows, int heads, int kv_heads, int dim, int vdim,
+                                      const float* sink, void* out, int rows, int heads, int kv_heads, int dim, int vdim,
                                       int window, int keep_first, float scale, float softcap, int own, int mode,
-                                      int pool, long pool_off, int maps, int dt, hipStream_t stream) {
+                                      int pool, long pool_off, int maps, const void* gate, long g_stride, int out_t,
+                                      int dt, hipStream_t stream) {
   if (rows <= 0) return 0;
   if ((own ? vdim : kv_heads * vdim) > 256 * WA_ACC || (size_t)dim * 4 > 32 * 1024 || heads % kv_heads) return 2;
   if (window < 1 || maps < 1 || kv_heads % maps || (maps > 1 && !own) || (pool > 0 && (keep_first || mode))) return 4;
@@ -1650,19 +1739,19 @@ VPSA_EXPORT int vpsa_window_attention(const void* q, long q_stride, const void* 
   SM_DISPATCH(dt, (window_attention_kernel<T><<<grid, 256, (size_t)dim * 4, stream>>>(
                       (const T*)q, q_stride, (const T*)cache, page_stride, block_tables, bt_stride, row_seq, positions,
                       sink, out, heads, kv_heads, dim, vdim, window, keep_first, scale, softcap, own, mode, pool, pool_off,
-                      maps)));
+                      maps, (const T*)gate, g_stride, out_t)));
   return 0;
 }
 
 // Value channels a workgroup of the matrix-core kernel takes (0: the shape is not tiled).
 static int window_chunk(int vall) {
-  for (int c = 512; c >= 128; c >>= 1)
+  for (int c : {512, 256, 128, 96, 64})
     if (vall % c == 0) return c;
   return 0;
 }
 
 VPSA_EXPORT int vpsa_window_mfma_supported(int heads, int kv_heads, int dim, int vdim, int own) {
-  return (dim == 64 || dim == 128) && window_chunk(own ? vdim : kv_heads * vdim) > 0 && heads % kv_heads == 0 &&
+  return (dim == 64 || dim == 96 || dim == 128) && window_chunk(own ? vdim : kv_heads * vdim) > 0 && heads % kv_heads == 0 &&
          heads / kv_heads <= 64;
 }
 
@@ -1673,10 +1762,11 @@ VPSA_EXPORT int vpsa_window_mfma_supported(int heads, int kv_heads, int dim, int
 
 template <int DIM, int VALL, int NSUB>
 static int launch_window_mfma(const void* q, long q_stride, const void* cache, long page_stride, const int* block_tables,
-                              int bt_stride, const int* tiles, const int* positions, const float* sink, float* out,
+                              int bt_stride, const int* tiles, const int* positions, const float* sink, void* out,
                               int n_tiles, int heads, int kv_heads, int window, int keep_first, float scale,
                               float softcap, int splits, float* ws_o, float* ws_ml, int n_chunks, int own, int mode,
-                              int pool, long pool_off, int maps, hipStream_t st) {
+                              int pool, long pool_off, int maps, const void* gate, long g_stride, int out_t,
+                              hipStream_t st) {
   constexpr int LDS = PAGE * (DIM * 2 + 16) + VALL * (PAGE * 2 + 16);
   static bool attr_set = false;
   if (!attr_set) {
@@ -1688,9 +1778,10 @@ static int launch_window_mfma(const void* q, long q_stride, const void* cache, l
   window_mfma_kernel<DIM, VALL, NSUB><<<dim3(n_tiles, kv_heads * n_chunks, splits), dim3(256), LDS, st>>>(
       (const uint16_t*)q, q_stride, (const uint16_t*)cache, page_stride, block_tables, bt_stride, tiles, positions, sink,
       out, heads, kv_heads, window, keep_first, scale, softcap, splits, ws_o, ws_ml, n_chunks, own, mode, pool, pool_off,
-      maps);
+      maps, (const uint16_t*)gate, g_stride, out_t);
   if (splits > 1)  // decode rows only: row r of the launch is row r of out
-    window_merge_kernel<<<n_tiles * heads, 128, 0, st>>>(ws_o, ws_ml, sink, out, heads, VALL * n_chunks, splits);
+    window_merge_kernel<<<n_tiles * heads, 128, 0, st>>>(ws_o, ws_ml, sink, out, heads, VALL * n_chunks, splits,
+                                                         (const uint16_t*)gate, g_stride, out_t);
   return 0;
 }
 
@@ -1701,11 +1792,13 @@ VPSA_EXPORT int vpsa_window_tile_slots() { return 64 * WINDOW_PREFILL_SUB; }
 // nullptr: n_tiles decode rows, row r = sequence r at positions[r].
 VPSA_EXPORT int vpsa_window_attention_mfma(const void* q, long q_stride, const void* cache, long page_stride,
                                            const int* block_tables, int bt_stride, const int* tiles,
-                                           const int* positions, const float* sink, float* out, int n_tiles, int heads,
+                                           const int* positions, const float* sink, void* out, int n_tiles, int heads,
                                            int kv_heads, int dim, int vdim, int window, int keep_first, float scale,
                                            float softcap, int splits, float* ws_o, float* ws_ml, int own, int mode,
-                                           int pool, long pool_off, int maps, hipStream_t stream) {
+                                           int pool, long pool_off, int maps, const void* gate, long g_stride,
+                                           int out_t, hipStream_t stream) {
   if (n_tiles <= 0) return 0;
+  if (q_stride & 7) return 5;
   if (window < 1 || maps < 1 || kv_heads % maps || (maps > 1 && !own) || (pool > 0 && (keep_first || mode))) return 4;
   if (!vpsa_window_mfma_supported(heads, kv_heads, dim, vdim, own)) return 2;
   if (splits < 1 || (splits > 1 && (tiles || !ws_o || !ws_ml))) return 3;  // splits are for decode rows
@@ -1716,12 +1809,16 @@ VPSA_EXPORT int vpsa_window_attention_mfma(const void* q, long q_stride, const v
       return launch_window_mfma<D, V, WINDOW_PREFILL_SUB>(q, q_stride, cache, page_stride, block_tables, bt_stride,    \
                                                           tiles, positions, sink, out, n_tiles, heads, kv_heads,      \
                                                           window, keep_first, scale, softcap, splits, ws_o, ws_ml,     \
-                                                          n_chunks, own, mode, pool, pool_off, maps, stream);         \
+                                                          n_chunks, own, mode, pool, pool_off, maps, gate, g_stride,  \
+                                                          out_t, stream);                                             \
     return launch_window_mfma<D, V, 1>(q, q_stride, cache, page_stride, block_tables, bt_stride, tiles, positions,     \
                                        sink, out, n_tiles, heads, kv_heads, window, keep_first, scale, softcap,       \
-                                       splits, ws_o, ws_ml, n_chunks, own, mode, pool, pool_off, maps, stream);       \
+                                       splits, ws_o, ws_ml, n_chunks, own, mode, pool, pool_off, maps, gate,          \
+                                       g_stride, out_t, stream);                                                      \
   }
-  WM(64, 128) WM(64, 256) WM(64, 512) WM(128, 128) WM(128, 256) WM(128, 512)
+#define WM_ALL(D) WM(D, 64) WM(D, 96) WM(D, 128) WM(D, 256) WM(D, 512)
+  WM_ALL(64) WM_ALL(96) WM_ALL(128)
+#undef WM_ALL
 #undef WM
   return 2;
 }

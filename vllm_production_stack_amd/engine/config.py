@@ -36,6 +36,7 @@ class LatentMixerSpec:
     sink: bool = True          # a learned per-head logit in the softmax denominator
     out_gate: bool = True      # head outputs times sigmoid(W_g h)
     rope_layout: str = "pairs"  # checkpoint order of the rotated channels: "pairs" (2 i, 2 i + 1) or "half" (i, i + dims / 2)
+    window: int = 0            # > 0: a position sees itself and the window - 1 positions before it, 0: all before it
 
     @property
     def entry(self) -> int:    # cached values per token
@@ -72,10 +73,11 @@ class FeedForwardSpec:
     kind: str = "dense"
     ff: int = 0
     act: str = "relu_sq"       # relu_sq | xielu (two learned curvatures, see ops.xielu) | poly_norm (four learned
-                               # numbers, see ops.poly_norm) | gelu_tanh | silu (gated units)
+                               # numbers, see ops.poly_norm) | gelu_tanh | silu | glu_clamp (gated units)
     gated: bool = False        # down(act(gate x) * (up x)) instead of down(act(up x))
     router: str = "sigmoid"    # sigmoid: as described above | softmax: softmax scores, a learned selection bias,
-                               # a group scores its largest biased score, weights = scores, not renormalised
+                               # a group scores its largest biased score, weights = scores, not renormalised |
+                               # softmax_top: the largest logits, weights = the softmax over the chosen ones alone
     identity: int = 0          # softmax router: extra outputs whose "expert" returns the token itself
     experts: int = 0
     top: int = 0
@@ -87,6 +89,7 @@ class FeedForwardSpec:
     limit: float = 0.0
     shared_ff: int = 0
     shared_limit: float = 0.0
+    shared_gate: bool = True   # False: the shared unit's output is added as it is
 
 
 @dataclass(frozen=True)
@@ -94,6 +97,7 @@ class LayerSpec:
     type: str
     mixer: LatentMixerSpec
     mlp: FeedForwardSpec | None = None
+    weights_of: int | None = None   # the layer whose tensors this one runs on, with cache entries of its own
 
 
 @dataclass(frozen=True)
@@ -294,6 +298,31 @@ class NormedAttentionSpec:
     def weight_count(self, width: int) -> int:
         n = width * self.heads * (self.dim + self.vdim) + self.heads * self.vdim * width
         return n + (width * self.kv_heads * (self.dim + self.vdim) if self.kv_from is None else 0)
+
+
+@dataclass(frozen=True)
+class SlidingAttentionSpec:
+    """Grouped-query softmax attention without rotation over a sliding window of ``window`` positions.  ``unit_sink``:
+    the softmax denominator is 1 + sum exp(s) (a sink of score 0 without a value).  ``head_gate``: a head's output is
+    multiplied by one number, sigmoid((W_g h)_head)."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    window: int
+    scale: float
+    unit_sink: bool = True
+    head_gate: bool = True
+
+    def cache_elems(self) -> int:        # per token: keys and values of every KV head
+        return self.kv_heads * (self.dim + self.vdim)
+
+    def weight_count(self, width: int) -> int:
+        n = width * (self.heads * self.dim + self.kv_heads * (self.dim + self.vdim)) + self.heads * self.vdim * width
+        return n + (width * self.heads if self.head_gate else 0)
+
+    def token_flops(self) -> float:      # a full window
+        return 2.0 * self.heads * (self.dim + self.vdim) * self.window
 
 
 @dataclass(frozen=True)
@@ -536,6 +565,78 @@ def zupilorn_config(name: str, vocab: int, width: int, layers: list[dict], logit
         bos_token_id=0, eos_token_id=-1)  # the design names no special tokens
 
 
+def guzovik_layers(layers: list[dict]) -> tuple:
+    """The ``layers`` list of a Guzovik config.json -> layer specs."""
+
+    def parse(i: int, entry: dict) -> tuple:
+        m = entry["mixer"]
+        kind = entry["type"]
+        if kind == "attention":
+            mixer = SlidingAttentionSpec(
+                heads=int(m["heads"]), kv_heads=int(m["kv_heads"]), dim=int(m["dim"]), vdim=int(m["vdim"]),
+                window=int(m["mask"]["size"]), scale=float(m["scale"]))
+            _positive(i, heads=mixer.heads, kv_heads=mixer.kv_heads, dim=mixer.dim, vdim=mixer.vdim, window=mixer.window)
+            if mixer.heads % mixer.kv_heads:
+                raise ValueError(f"layer {i}: heads must be a multiple of kv_heads")
+        elif kind == "latent_attention":
+            rot = m["rot"]
+            mixer = LatentMixerSpec(
+                heads=int(m["heads"]), dim=int(m["dim"]), rot_dim=int(m["rot_dim"]), vdim=int(m["vdim"]),
+                kv_rank=int(m["kv_rank"]), q_rank=0, rope_base=float(rot["base"]),
+                rope_dims=int(rot.get("dims", m["rot_dim"])), scale=float(m["scale"]), sink=False, out_gate=False,
+                window=int(m["mask"]["size"]))
+            _positive(i, heads=mixer.heads, dim=mixer.dim, rot_dim=mixer.rot_dim, vdim=mixer.vdim, kv_rank=mixer.kv_rank,
+                      window=mixer.window)
+            if mixer.rope_dims % 2 or not 0 < mixer.rope_dims <= mixer.rot_dim:
+                raise ValueError(f"layer {i}: rotary dims must be even and within rot_dim")
+        else:
+            raise ValueError(f"layer {i}: unknown mixer type {kind!r}")
+        f = entry.get("mlp")
+        mlp = None
+        if f is not None:
+            if f["kind"] == "dense":
+                mlp = FeedForwardSpec(kind="dense", ff=int(f["ff"]), act="glu_clamp", gated=True, limit=float(f["limit"]))
+                if mlp.limit <= 0:
+                    raise ValueError(f"layer {i}: the limit must be positive")
+            elif f["kind"] == "moe":
+                r, sh = f["router"], f.get("shared")
+                mlp = FeedForwardSpec(kind="moe", ff=int(f["expert"]["ff"]), act="silu", gated=True, router="softmax_top",
+                                      experts=int(r["experts"]), top=int(r["top"]), shared_ff=int(sh["ff"]) if sh else 0,
+                                      shared_gate=False)
+                if not 1 <= mlp.top <= mlp.experts:
+                    raise ValueError(f"layer {i}: 1 <= top <= experts is required")
+            else:
+                raise ValueError(f"layer {i}: unknown feed-forward kind {f['kind']!r}")
+            _positive(i, ff=mlp.ff)
+        return kind, mixer, mlp
+
+    parsed = [parse(i, entry) for i, entry in enumerate(layers)]
+    out = []
+    for i, entry in enumerate(layers):
+        src, seen = i, {i}
+        while layers[src].get("weights_of") is not None:   # a layer may name one that itself runs on another's tensors
+            src = int(layers[src]["weights_of"])
+            if not 0 <= src < len(layers) or src in seen:
+                raise ValueError(f"layer {i}: weights_of must lead to another layer that has tensors")
+            seen.add(src)
+        if parsed[src] != parsed[i]:
+            raise ValueError(f"layer {i}: layer {src}, whose tensors it runs on, has another shape")
+        out.append(LayerSpec(*parsed[i], weights_of=None if src == i else src))
+    return tuple(out)
+
+
+def guzovik_config(name: str, vocab: int, width: int, layers: list[dict], embedding_scale: float = 1.0,
+                   norm_eps: float = 1e-5, max_position_embeddings: int = 32768) -> "ModelConfig":
+    specs = guzovik_layers(layers)
+    return ModelConfig(
+        name=name, architecture="guzovik", vocab_size=int(vocab), hidden_size=int(width),
+        intermediate_size=max([s.mlp.ff for s in specs if s.mlp] + [0]), num_layers=len(specs),
+        num_heads=max(s.mixer.heads for s in specs), num_kv_heads=max([getattr(s.mixer, "kv_heads", 1) for s in specs]),
+        head_dim=max(s.mixer.dim + getattr(s.mixer, "rot_dim", 0) for s in specs), norm_eps=float(norm_eps),
+        max_position_embeddings=max_position_embeddings, embedding_scale=float(embedding_scale), layer_specs=specs,
+        bos_token_id=0, eos_token_id=-1)  # the design names no special tokens
+
+
 def _rotary(rot: dict, layout: str) -> RotarySpec:
     sc = rot.get("scaling")
     scaling = None if not sc else (float(sc["factor"]), float(sc["original"]), float(sc["fast"]), float(sc["slow"]))
@@ -647,7 +748,8 @@ def zururax_config(name: str, vocab: int, width: int, layers: list[dict], embedd
 @dataclass
 class ModelConfig:
     name: str = "tiny-llama"
-    architecture: str = "llama"  # llama | mixtral | opt | gpt2 | zururax | revelix | pelatar | zetalorn | zupilorn
+    # llama | mixtral | opt | gpt2 | zururax | revelix | pelatar | zetalorn | zupilorn | guzovik
+    architecture: str = "llama"
     vocab_size: int = 512
     hidden_size: int = 256
     intermediate_size: int = 512
@@ -707,7 +809,10 @@ class ModelConfig:
                 m, f = s.mixer, s.mlp
                 gemm += m.weight_count(h)
                 if isinstance(m, LatentMixerSpec):
-                    pair += m.heads * (m.entry + m.kv_rank)
+                    if m.window:
+                        gemm += m.heads * (m.entry + m.kv_rank) * m.window
+                    else:
+                        pair += m.heads * (m.entry + m.kv_rank)
                 elif isinstance(m, NormedAttentionSpec):
                     pair += m.heads * (m.dim + m.vdim)
                 else:  # recurrences cost per token, a windowed softmax at most its window per token
@@ -730,6 +835,8 @@ class ModelConfig:
             n = self.vocab_size * h * (1 if self.tie_word_embeddings else 2)
             for s in self.layer_specs:
                 m, f = s.mixer, s.mlp
+                if s.weights_of is not None:
+                    continue
                 n += m.weight_count(h)
                 if f is not None:
                     n += ((3 if f.gated else 2) * h * f.ff if f.kind == "dense"
@@ -1007,6 +1114,45 @@ PRESETS["tiny-zupilorn"] = zupilorn_config(
 PRESETS["zupilorn-bench"] = zupilorn_config("zupilorn-bench", 32000, 2048, zupilorn_stack(2048, 16, 5120, 16, 1024, 4, 2),
                                             logit_softcap=30.0)
 
+
+
+def _gz_attention(heads, kv_heads, dim, vdim, window, mlp):
+    return {"type": "attention", "mlp": mlp,
+            "mixer": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "mask": {"size": window},
+                      "scale": dim ** -0.5}}
+
+
+def _gz_latent(heads, dim, rot_dim, vdim, kv_rank, window, mlp, base=10000.0):
+    return {"type": "latent_attention", "mlp": mlp,
+            "mixer": {"heads": heads, "dim": dim, "rot_dim": rot_dim, "vdim": vdim, "kv_rank": kv_rank,
+                      "mask": {"size": window}, "rot": {"base": base, "dims": rot_dim}, "scale": (dim + rot_dim) ** -0.5}}
+
+
+def _gz_moe(ff, experts, top, shared):
+    return {"kind": "moe", "expert": {"ff": ff}, "router": {"experts": experts, "top": top},
+            "shared": {"ff": shared} if shared else None}
+
+
+def guzovik_stack(heads, ff, experts, unit_ff, top, shared, window=1024, latent_window=2048):
+    """Layer list of a Guzovik at random weights: a sliding attention layer with a dense feed-forward, one and a latent
+    layer with routed units, and the second layer's tensors once more."""
+    moe = _gz_moe(unit_ff, experts, top, shared)
+    out = [_gz_attention(heads, max(1, heads // 4), 128, 128, window, {"kind": "dense", "ff": ff, "limit": 7.0}),
+           _gz_attention(heads, max(1, heads // 4), 128, 128, window, moe),
+           _gz_latent(heads, 128, 64, 128, 512, latent_window, moe)]
+    return out + [{**out[1], "weights_of": 1}]
+
+
+# Guzovik at random weights: a small one for smoke runs, and one with layer shapes of a 2048-wide model
+PRESETS["tiny-guzovik"] = guzovik_config(
+    "tiny-guzovik", 512, 192,
+    [_gz_latent(3, 24, 32, 40, 64, 100, _gz_moe(64, 6, 2, 96), base=5000.0),
+     _gz_attention(6, 2, 64, 128, 70, {"kind": "dense", "ff": 320, "limit": 2.0}),
+     _gz_attention(4, 4, 32, 48, 130, None), {**_gz_attention(6, 2, 64, 128, 70, {"kind": "dense", "ff": 320, "limit": 2.0}),
+                                              "weights_of": 1}],
+    embedding_scale=8.0, max_position_embeddings=4096)
+PRESETS["guzovik-bench"] = guzovik_config("guzovik-bench", 32000, 2048, guzovik_stack(16, 5120, 16, 1024, 4, 1024))
+
 _ALIASES = {
     "meta-llama/meta-llama-3-8b": "llama-3-8b",
     "meta-llama/meta-llama-3-8b-instruct": "llama-3-8b",
@@ -1049,6 +1195,11 @@ def _from_hf_config(cfg: dict[str, Any], name: str) -> ModelConfig:
         return zupilorn_config(name, cfg["vocab"], cfg["width"], cfg["layers"], logit_softcap=cfg.get("logit_softcap"),
                                norm_eps=(cfg.get("norm") or {}).get("eps", 1e-5),
                                max_position_embeddings=int(cfg.get("max_positions", 32768)))
+    if str(cfg.get("architecture", "")).lower() == "guzovik":
+        return guzovik_config(name, cfg["vocab"], cfg["width"], cfg["layers"],
+                              embedding_scale=(cfg.get("embedding") or {}).get("scale", 1.0),
+                              norm_eps=(cfg.get("norm") or {}).get("eps", 1e-5),
+                              max_position_embeddings=int(cfg.get("max_positions", 32768)))
     if str(cfg.get("architecture", "")).lower() == "pelatar":
         return pelatar_config(name, cfg["vocab"], cfg["width"], cfg["layers"],
                               norm_eps=(cfg.get("norm") or {}).get("eps", 1e-5),

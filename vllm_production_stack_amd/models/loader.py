@@ -17,6 +17,7 @@ from ..engine.config import ModelConfig
 from ..parallel.state import get_tp
 from .opt import OPTModel
 from .transformer import LayerWeights, TransformerModel
+from .guzovik import GuzovikModel
 from .pelatar import PelatarModel
 from .revelix import RevelixModel
 from .zetalorn import ZetalornModel
@@ -39,6 +40,8 @@ def build_model(cfg: ModelConfig, dtype: torch.dtype, device: torch.device, max_
         model = ZetalornModel(cfg, dtype, device, max_model_len)
     elif cfg.architecture == "zupilorn":
         model = ZupilornModel(cfg, dtype, device, max_model_len)
+    elif cfg.architecture == "guzovik":
+        model = GuzovikModel(cfg, dtype, device, max_model_len)
     else:
         model = TransformerModel(cfg, dtype, device, max_model_len, expert_parallel=expert_parallel)
     has_weights = ckpt_dir is not None and any(Path(ckpt_dir).glob("*.safetensors"))
@@ -78,6 +81,8 @@ def load_hf_weights(model, ckpt_dir: Path) -> None:
         _load_zetalorn(model, ckpt_dir)
     elif isinstance(model, ZupilornModel):
         _load_zupilorn(model, ckpt_dir)
+    elif isinstance(model, GuzovikModel):
+        _load_guzovik(model, ckpt_dir)
     else:
         _load_llama(model, ckpt_dir)
 
@@ -807,6 +812,88 @@ def _load_zupilorn(model: ZupilornModel, ckpt_dir: Path) -> None:
         if name not in places:
             raise ValueError(f"unexpected tensor {name!r}")
         places[name](t, name)
+        seen.add(name)
+    if set(places) - seen:
+        raise ValueError(f"checkpoint lacks {sorted(set(places) - seen)[:8]}")
+
+
+def _load_guzovik(model: GuzovikModel, ckpt_dir: Path) -> None:
+    """Guzovik checkpoints: ``embed``, ``head``, ``final.norm``; per layer that has tensors of its own ``l<i>.norm1|norm1b|
+    ls1`` (and, with a feed-forward, ``norm2|norm2b|ls2``), ``l<i>.mix.{q, k, v, g, o}`` (attention) or
+    ``l<i>.mix.{q, dkv, dkv.norm, uk, uv, o}`` (latent attention), ``l<i>.mlp.{gate, up, down}`` or ``l<i>.mlp.router``,
+    ``l<i>.mlp.e<j>.{gate, up, down}`` and ``l<i>.mlp.shared.{gate, up, down}``.  Linear weights are [out, in]; a mixer's
+    input projections are fused row-wise here, the units stacked.  The model's norms are stored around zero (gain
+    1 + w), the latent's as it is; a layer scale is multiplied into the gain of the norm it follows.  Every tensor the
+    model holds must be found, and every tensor of the file must have a place."""
+    from ..engine.config import SlidingAttentionSpec
+
+    def same_shape(dst, src, what: str) -> None:
+        if tuple(dst.shape) != tuple(src.shape):
+            raise ValueError(f"{what}: checkpoint shape {tuple(src.shape)}, model expects {tuple(dst.shape)}")
+
+    def put(dst, src, what):
+        same_shape(dst, src, what)
+        dst.copy_(src.to(dst.dtype))
+
+    def put_gain(dst, src, what):
+        put(dst, 1.0 + src.float(), what)
+
+    def times_gain(dst, src, what):
+        same_shape(dst, src, what)
+        dst.mul_(1.0 + src.float().to(dst.device))
+
+    def times(dst, src, what):
+        same_shape(dst, src, what)
+        dst.mul_(src.float().to(dst.device))
+
+    def put_heads(dst, src, what):
+        if tuple(src.shape) != (dst.shape[0] * dst.shape[2], dst.shape[1]):
+            raise ValueError(f"{what}: checkpoint shape {tuple(src.shape)}, model expects "
+                             f"{(dst.shape[0] * dst.shape[2], dst.shape[1])}")
+        put(dst, heads_transposed(src, dst.shape[0]), what)
+
+    def unit_places(name: str, w13, w2) -> dict:
+        ff = w2.shape[1]
+        return {f"{name}.gate": (put, w13[:ff]), f"{name}.up": (put, w13[ff:]), f"{name}.down": (put, w2)}
+
+    def layer_places(lw) -> dict:
+        m, f = lw.spec.mixer, lw.spec.mlp
+        rows = model.in_rows(m)
+        for post in (lw.post1, lw.post2):
+            if post is not None:
+                post.fill_(1.0)   # two tensors of the file multiply into it, in any order
+        out = {"norm1": (put_gain, lw.norm1), "norm1b": (times_gain, lw.post1), "ls1": (times, lw.post1),
+               "mix.o": (put, lw.w_o), "mix.q": (put, lw.w_in[slice(*rows["q"])])}
+        if isinstance(m, SlidingAttentionSpec):
+            for part in ("k", "v", "g"):
+                out[f"mix.{part}"] = (put, lw.w_in[slice(*rows[part])])
+        else:
+            out["mix.dkv"] = (put, lw.w_in[slice(*rows["dkv"])])
+            out["mix.dkv.norm"] = (put, lw.dkv_norm)
+            out["mix.uk"] = (put, lw.w_uk.view(m.heads * m.dim, m.kv_rank))
+            out["mix.uv"] = (put_heads, lw.w_uv)
+        if f is not None:
+            out.update({"norm2": (put_gain, lw.norm2), "norm2b": (times_gain, lw.post2), "ls2": (times, lw.post2)})
+            if f.kind == "dense":
+                out.update(unit_places("mlp", lw.w_gu, lw.w_down))
+            else:
+                out["mlp.router"] = (put, lw.router)
+                for e in range(f.experts):
+                    out.update(unit_places(f"mlp.e{e}", lw.w13[e], lw.w2[e]))
+                if f.shared_ff:
+                    out.update(unit_places("mlp.shared", lw.w_sh13, lw.w_sh2))
+        return out
+
+    places: dict = {"embed": (put, model.embed), "head": (put, model.lm_head), "final.norm": (put_gain, model.norm)}
+    owners = [i for i, s in enumerate(model.specs) if s.weights_of is None]
+    for i, lw in zip(owners, model.layers):
+        places.update({f"l{i}.{sub}": place for sub, place in layer_places(lw).items()})
+    seen = set()
+    for name, t in _iter_safetensors(ckpt_dir):
+        if name not in places or name in seen:
+            raise ValueError(f"unexpected tensor {name!r}")
+        how, dst = places[name]
+        how(dst, t, name)
         seen.add(name)
     if set(places) - seen:
         raise ValueError(f"checkpoint lacks {sorted(set(places) - seen)[:8]}")

@@ -99,8 +99,9 @@ class PelatarModel:
     def graph_capturable(self) -> bool:
         """Decode steps can be captured when no layer's mixture falls back to the per-unit loop, which reads
         the row counts on the host (shapes the grouped GEMMs do not tile, fp32)."""
+        probe = torch.empty((1, self.cfg.hidden_size), dtype=self.dtype, device=self.device)
         return self.dtype == torch.bfloat16 and self.device.type == "cuda" and all(
-            lw.w13 is None or self._grouped(lw) for lw in self.layers)
+            lw.w13 is None or ops.moe_units_grouped(probe, lw.w13, lw.w2) for lw in self.layers)
 
     # ------------------------------------------------------------------ stores
     def kv_page_shape(self) -> tuple:
@@ -278,12 +279,6 @@ class PelatarModel:
         return ops.linear(y, lw.w_o)
 
     # ------------------------------------------------------------------ feed-forwards
-    def _grouped(self, lw: PelatarLayer) -> bool:
-        """Do the grouped matrix-core GEMMs take this layer's units?"""
-        return (self.device.type == "cuda" and self.dtype == torch.bfloat16
-                and ops.grouped_gemm_supported(lw.w13.shape[1], lw.w13.shape[2], True)
-                and ops.grouped_gemm_supported(lw.w2.shape[1], lw.w2.shape[2]))
-
     def _moe(self, lw: PelatarLayer, x: torch.Tensor, h: torch.Tensor) -> torch.Tensor:
         """The mixture's output for rows h, fp32."""
         f: FeedForwardSpec = lw.spec.mlp
@@ -292,22 +287,7 @@ class PelatarModel:
         w, ids, gate = ops.route_softmax(logits, f.experts + f.identity, f.experts, f.groups, f.keep, f.top,
                                          lw.correction, 1.0, park_in_bucket=True)
         out = torch.zeros((t, width), dtype=torch.float32, device=h.device)
-        bucket = f.identity > 0
-        if self._grouped(lw):
-            if t <= ops.MOE_MFMA_MAX_TOKENS and ops.moe_mfma_supported(width, f.ff):
-                ys, pos = ops.moe_experts_grouped(h, lw.w13, lw.w2, ids, w, foreign=bucket, combine=False)
-            else:
-                ys, pos = ops.moe_experts_prefill(h, lw.w13, lw.w2, ids, w, foreign=bucket, combine=False)
-        else:
-            # the CPU, fp32, and shapes the grouped kernels do not tile: unit by unit on the sorted rows
-            offsets, pos, sorted_tok = ops.moe_align(ids, f.experts + (1 if bucket else 0))
-            xs = ops.gather_rows(h, sorted_tok)
-            ys = torch.empty((t * f.top, width), dtype=h.dtype, device=h.device)
-            off = offsets.tolist()
-            for e in range(f.experts):
-                a, b = off[e], off[e + 1]
-                if b > a:
-                    torch.matmul(ops.glu_act(F.linear(xs[a:b], lw.w13[e]), f.act), lw.w2[e].t(), out=ys[a:b])
+        ys, pos = ops.moe_units(h, lw.w13, lw.w2, ids, f.act, bucket=f.identity > 0)
         return ops.moe_finish(out, ys, w, pos, h if gate is not None else None, gate)
 
     # ------------------------------------------------------------------ forward

@@ -44,6 +44,7 @@ def _kernels():
             "vpsa_add_dyt", "vpsa_recurrent_scan", "vpsa_head_rms", "vpsa_short_conv_qkv", "vpsa_window_attention",
             "vpsa_mix_heads", "vpsa_xielu", "vpsa_window_mfma_supported", "vpsa_window_attention_mfma", "vpsa_window_tile_slots",
             "vpsa_gated_add_rmsnorm", "vpsa_pool_blocks", "vpsa_diff_heads",
+            "vpsa_window_kv_write",
             "vpsa_embed_rmsnorm", "vpsa_depth_mix_rmsnorm", "vpsa_poly_norm", "vpsa_soft_cap", "vpsa_mingru",
         ):
             getattr(lib, name).restype = c_int
@@ -1351,10 +1352,10 @@ def lora_expand(h, bs, slots, y, r_pad):
 from .latent import (add_rms_norm, build_latent_tiles, embed_scale, gate_up_glu_clamp, gather_rows, glu_clamp,  # noqa: E402,F401
                      depth_mix_rms_norm, embed_rms_norm, moe_glu, poly_norm, soft_cap, up_poly_norm,
                      gate_up_act, gated_add_rms_norm, glu_act, rms_norm_add, route_softmax,
-                     group_topk, latent_attention, moe_glu_grouped, moe_glu_grouped_supported, up_relu_sq,
+                     group_topk, latent_attention, moe_glu_grouped, moe_glu_grouped_supported, moe_units, moe_units_grouped, up_relu_sq,
                      latent_kv_write, latent_mfma_supported, latent_tile_kernel_takes, moe_finish, relu_sq, rms_norm_rows, rope_pairs, sigmoid_gate)
 
 # --------------------------------------------------------------------------- recurrent mixers, windowed attention, Dynamic Tanh
 from .seqmix import (add_dyt_norm, build_gru_pieces, build_scan_pieces, mingru_scan, build_window_tiles, head_rms_norm, mix_heads, recurrent_scan, short_conv_qkv,  # noqa: E402,F401
                      diff_heads, gla_prepare, head_finish, mlstm_prepare, pool_blocks, prepared_scan, qk_norm_write, scan_state_cols,
-                     up_xielu, window_attention, window_cache_elems, window_decode_splits, window_mfma_supported, xielu)
+                     up_xielu, window_attention, window_cache_elems, window_decode_splits, window_kv_write, window_mfma_supported, xielu)

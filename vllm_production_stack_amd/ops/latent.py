@@ -232,6 +232,7 @@ def rope_pairs(q, positions, cos_sin, col0: int, rot_dims: int):
                                           c_int(rot_dims), c_int(_dt(q)), o._stream()), "rope_pairs")
 
 
+NO_WINDOW = 1 << 30     # a window no context reaches: plain causal attention
 LATENT_TILE_SLOTS = 64  # (token, head) pairs of one tile of the matrix-core kernel
 LATENT_MFMA = True      # False: every call takes the plain kernel (A/B runs, tests of the plain kernel)
 
@@ -280,24 +281,26 @@ def latent_tile_kernel_takes(q_lat, q_rot, pool, out) -> bool:
 
 
 def latent_attention(q_lat, q_rot, pool, offset: int, block_tables, row_seq, positions, sink, scale: float, out=None,
-                     tiles=None, splits: int = 1):
+                     tiles=None, splits: int = 1, window: int = NO_WINDOW):
     """Causal attention of query rows over their sequences' cache entries, in latent space.
 
     q_lat [T, heads, rank] and q_rot [T, heads, rot] (views with contiguous last dim); row ``i``
     belongs to sequence ``row_seq[i]`` (``None``: row i is sequence i, a decode batch) whose pages are
-    ``block_tables[seq]`` and sees entries 0 .. positions[i].  ``sink`` [heads] fp32 or None: a logit
+    ``block_tables[seq]`` and sees entries 0 .. positions[i], of these the last ``window``.  ``sink`` [heads] fp32 or None: a logit
     that joins the softmax denominator only.  Returns [T, heads, rank].
 
     bf16 entries of a shape the matrix-core kernel tiles take it: decode batches as they are (with
     ``splits`` key ranges per row, merged by a second launch), prefill rows when ``tiles`` (the device
     copy of ``build_latent_tiles``) describes them.  Everything else takes the plain kernel."""
     t, heads, rank = q_lat.shape
+    assert 1 <= window <= NO_WINDOW
     if out is None:
         out = torch.empty((t, heads, rank), dtype=q_lat.dtype, device=q_lat.device)
     if t == 0:
         return out
     if not q_lat.is_cuda:
-        return reference.latent_attention(q_lat, q_rot, pool, offset, block_tables, row_seq, positions, sink, scale, out)
+        return reference.latent_attention(q_lat, q_rot, pool, offset, block_tables, row_seq, positions, sink, scale, out,
+                                          window)
     o = _ops()
     rot = q_rot.shape[2]
     _f32(sink)
@@ -320,14 +323,14 @@ def latent_attention(q_lat, q_rot, pool, offset: int, block_tables, row_seq, pos
             c_long(q_rot.stride(1)), _layer_base(pool, offset, rank + rot), c_long(pool.stride(0)), o._p(block_tables),
             c_int(block_tables.stride(0)), o._p(tiles), o._p(positions), c_int(n_tiles), c_int(heads), o._p(sink),
             o._p(out), c_long(out.stride(0)), c_long(out.stride(1)), c_int(rank), c_int(rot), c_float(scale),
-            c_int(splits), o._p(ws_o), o._p(ws_ml), o._stream()), "latent_attention_mfma")
+            c_int(window), c_int(splits), o._p(ws_o), o._p(ws_ml), o._stream()), "latent_attention_mfma")
         return out
     o._check(o._kernels().vpsa_latent_attention(
         o._p(q_lat), c_long(q_lat.stride(0)), c_long(q_lat.stride(1)), o._p(q_rot), c_long(q_rot.stride(0)),
         c_long(q_rot.stride(1)), _layer_base(pool, offset, rank + rot), c_long(pool.stride(0)), o._p(block_tables),
         c_int(block_tables.stride(0)), o._p(row_seq), o._p(positions), o._p(sink), o._p(out), c_long(out.stride(0)),
         c_long(out.stride(1)), c_int(t), c_int(heads), c_int(rank), c_int(rot), c_float(scale),
-        c_int(dt), o._stream()), "latent_attention")
+        c_int(window), c_int(dt), o._stream()), "latent_attention")
     return out
 
 
@@ -428,16 +431,19 @@ def gate_up_act(x, w_gate_up, act: str, packed=None):
 
 
 def route_softmax(logits, n: int, experts: int, groups: int, keep: int, topk: int, bias=None, route_scale: float = 1.0,
-                  park_in_bucket: bool = True):
+                  park_in_bucket: bool = True, normalize: bool = False):
     """Router logits fp32 [T, >= n] -> (weights fp32 [T, topk], ids int32 [T, topk], gate fp32 [T] or None).
     Scores are the softmax over all ``n`` outputs; an output is chosen by score + ``bias`` (fp32 [n]) and
     weighted by the score alone (times ``route_scale``, not renormalised).  Outputs form ``groups`` equal
     runs of neighbours, a group scores its largest biased score, and only outputs of the ``keep`` best
     groups can be chosen.  Outputs ``experts .. n`` are identity experts (their output is the token itself):
     a chosen one leaves the pair list (weight 0, id ``experts`` with ``park_in_bucket``, a bucket that sorting
-    kernels put behind the last expert and no product visits, else id 0) and its score is added to ``gate``."""
+    kernels put behind the last expert and no product visits, else id 0) and its score is added to ``gate``.
+    ``normalize`` (without identity experts): the chosen scores are divided by their sum, so that the weights are the
+    softmax over the chosen logits alone."""
+    assert not (normalize and experts < n)
     if not logits.is_cuda:
-        return reference.route_softmax(logits, n, experts, groups, keep, topk, bias, route_scale, park_in_bucket)
+        return reference.route_softmax(logits, n, experts, groups, keep, topk, bias, route_scale, park_in_bucket, normalize)
     o = _ops()
     _f32(logits, bias)
     t = logits.shape[0]
@@ -447,7 +453,7 @@ def route_softmax(logits, n: int, experts: int, groups: int, keep: int, topk: in
     o._check(o._kernels().vpsa_route_softmax(o._p(logits), c_int(logits.shape[1]), o._p(bias), o._p(w), o._p(ids),
                                              o._p(gate), c_int(t), c_int(n), c_int(experts), c_int(groups), c_int(keep),
                                              c_int(topk), c_float(route_scale), c_int(experts if park_in_bucket else 0),
-                                             o._stream()), "route_softmax")
+                                             c_int(1 if normalize else 0), o._stream()), "route_softmax")
     return w, ids, gate
 
 
@@ -526,6 +532,37 @@ def up_relu_sq(x, w_up):
 def up_poly_norm(x, w_up, act, eps: float):
     """poly_norm(x @ W.T): the projection, then one pass over its rows (the norms need whole rows)."""
     return poly_norm(_ops().linear(x, w_up), act, eps)
+
+
+def moe_units_grouped(x, w13, w2) -> bool:
+    """Do the grouped matrix-core GEMMs take a mixture of silu gated units of this shape?"""
+    o = _ops()
+    return (x.is_cuda and x.dtype == torch.bfloat16 and o.grouped_gemm_supported(w13.shape[1], w13.shape[2], True)
+            and o.grouped_gemm_supported(w2.shape[1], w2.shape[2]))
+
+
+def moe_units(x, w13, w2, ids, act: str = "silu", bucket: bool = False):
+    """Gated units act(gate x) * (up x) of a mixture over its (token, unit) pairs.  silu units of a shape the grouped
+    matrix-core GEMMs tile: decode-sized batches stream each routed unit's weights once against its few tokens,
+    larger ones run the grouped prefill GEMM, both on device-sorted pairs with no host synchronisation (HIP-graph
+    capturable).  Everything else (the CPU, fp32, other widths) runs unit by unit on the sorted rows, which reads the row
+    counts on the host.  ``bucket``: ids may equal the unit count, pairs that no unit sees (they sort last).
+    Returns (y [T * K, hidden] in sorted order, pos [T * K]: the sorted row of pair t * K + k)."""
+    o = _ops()
+    t, k = ids.shape
+    if act == "silu" and moe_units_grouped(x, w13, w2):
+        if t <= o.MOE_MFMA_MAX_TOKENS and o.moe_mfma_supported(x.shape[1], w2.shape[2]):
+            return o.moe_experts_grouped(x, w13, w2, ids, None, foreign=bucket, combine=False)
+        return o.moe_experts_prefill(x, w13, w2, ids, None, foreign=bucket, combine=False)
+    offsets, pos, sorted_tok = o.moe_align(ids, w13.shape[0] + (1 if bucket else 0))
+    xs = gather_rows(x, sorted_tok)
+    ys = torch.empty((t * k, x.shape[1]), dtype=x.dtype, device=x.device)
+    off = offsets.tolist()
+    for e in range(w13.shape[0]):
+        a, b = off[e], off[e + 1]
+        if b > a:
+            torch.matmul(glu_act(torch.nn.functional.linear(xs[a:b], w13[e]), act), w2[e].t(), out=ys[a:b])
+    return ys, pos
 
 
 def moe_glu_grouped_supported(x, w13, w2) -> bool:

@@ -429,7 +429,7 @@ def glu_act(x, act):
     return (a * u).to(x.dtype)
 
 
-def route_softmax(logits, n, experts, groups, keep, topk, bias, route_scale, park_in_bucket):
+def route_softmax(logits, n, experts, groups, keep, topk, bias, route_scale, park_in_bucket, normalize=False):
     t = logits.shape[0]
     s = torch.softmax(logits[:, :n].float(), dim=-1)
     c = s + bias if bias is not None else s.clone()
@@ -440,7 +440,10 @@ def route_softmax(logits, n, experts, groups, keep, topk, bias, route_scale, par
     allowed.scatter_(1, order, True)
     c = torch.where(allowed[:, :, None].expand(t, groups, per).reshape(t, n), c, torch.full_like(c, -math.inf))
     ids = torch.sort(c, dim=-1, descending=True, stable=True).indices[:, :topk]
-    w = s.gather(1, ids) * route_scale
+    w = s.gather(1, ids)
+    if normalize:
+        w = w / w.sum(-1, keepdim=True)
+    w = w * route_scale
     if experts == n:
         return w, ids.int(), None
     ident = ids >= experts
@@ -487,7 +490,7 @@ def rope_pairs(q, positions, cos_sin, col0, rot_dims):
     q[:, :, col0:col0 + rot_dims] = _rotate_pairs(part, cos_sin[positions.long()][:, None, :], rot_dims).to(q.dtype)
 
 
-def latent_attention(q_lat, q_rot, pool, offset, block_tables, row_seq, positions, sink, scale, out):
+def latent_attention(q_lat, q_rot, pool, offset, block_tables, row_seq, positions, sink, scale, out, window=1 << 30):
     t, heads, rank = q_lat.shape
     rot = q_rot.shape[2]
     view = latent_cache_view(pool, offset, rank + rot)
@@ -500,7 +503,8 @@ def latent_attention(q_lat, q_rot, pool, offset, block_tables, row_seq, position
         kv = view[pages].reshape(-1, rank + rot)[:ctx].float()
         q = torch.cat([q_lat[rows].float(), q_rot[rows].float()], dim=-1) * scale
         sc = torch.einsum("qhd,kd->qhk", q, kv)
-        sc = sc.masked_fill(torch.arange(ctx)[None, None, :] > pos[:, None, None], float("-inf"))
+        back = pos[:, None, None] - torch.arange(ctx)[None, None, :]
+        sc = sc.masked_fill((back < 0) | (back >= window), float("-inf"))
         m = sc.max(-1).values
         if sink is not None:
             m = torch.maximum(m, sink[None, :])
@@ -826,7 +830,7 @@ def short_conv_qkv(proj, conv_w, heads, kv_heads, dim, vdim, state, state_off, s
 
 
 def window_attention(q, pool, cache_off, kv_heads, vdim, block_tables, row_seq, positions, window, keep_first, scale,
-                     softcap, sink, out, own_values=False, mode=0, pool_block=0, pool_off=0, maps=1):
+                     softcap, sink, out, own_values=False, mode=0, pool_block=0, pool_off=0, maps=1, head_gate=None):
     t, heads, dim = q.shape
     kc, vc = window_cache_views(pool, cache_off, kv_heads, dim, vdim, kv_heads // maps)
     if pool_block:
@@ -856,11 +860,21 @@ def window_attention(q, pool, cache_off, kv_heads, vdim, block_tables, row_seq, 
             mx = torch.maximum(sc.max(-1).values, sink)
             e = torch.exp(sc - mx[:, None])
             w = e / (e.sum(-1) + torch.exp(sink - mx))[:, None]
+        if head_gate is not None:
+            w = w * torch.sigmoid(head_gate[r].float())[:, None]
         if own_values:
             out[r, :, 0] = torch.einsum("hk,khv->hv", w, vv.repeat_interleave(rep * maps, dim=1))
         else:
             out[r] = torch.einsum("hk,kgv->hgv", w, vv)
     return out
+
+
+def window_kv_write(k, v, slots, pool, cache_off, kv_heads, dim, vdim):
+    kc, vc = window_cache_views(pool, cache_off, kv_heads, dim, vdim)
+    ok = slots >= 0
+    pg, off = (slots[ok] // PAGE).long(), (slots[ok] % PAGE).long()
+    kc[pg, off] = k[ok].reshape(-1, kv_heads, dim).to(pool.dtype)
+    vc[pg, off] = v[ok].reshape(-1, kv_heads, vdim).to(pool.dtype)
 
 
 def mix_heads(u, talk, out_dtype):

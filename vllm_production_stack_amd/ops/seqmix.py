@@ -385,6 +385,24 @@ def qk_norm_write(proj, heads: int, kv_heads: int, dim: int, vdim: int, position
     return q
 
 
+def window_kv_write(proj, k_col: int, v_col: int, kv_heads: int, dim: int, vdim: int, slots, pool, cache_off: int):
+    """Keys and values of the step, column ranges of ``proj`` [T, cols] (heads side by side), to the paged cache at
+    ``slots`` (< 0: not cached) in the layout ``window_attention`` reads: what designs without a norm or a rotation on
+    q and k need (their attention reads q from the projection itself)."""
+    t = proj.shape[0]
+    nk, nv = kv_heads * dim, kv_heads * vdim
+    k, v = proj[:, k_col:k_col + nk], proj[:, v_col:v_col + nv]
+    if not proj.is_cuda:
+        return reference.window_kv_write(k, v, slots, pool, cache_off, kv_heads, dim, vdim)
+    o = _ops()
+    assert _rows(proj) and max(k_col + nk, v_col + nv) <= proj.shape[1]
+    assert slots.dtype == torch.int64 and slots.is_contiguous() and slots.numel() >= t
+    assert pool.dim() == 2 and pool.stride(1) == 1 and cache_off + window_cache_elems(kv_heads, dim, vdim) <= pool.shape[1]
+    o._check(o._kernels().vpsa_window_kv_write(o._p(k), o._p(v), c_long(proj.stride(0)), o._p(slots), _at(pool, cache_off),
+                                               c_long(pool.stride(0)), c_int(t), c_int(nk), c_int(nv),
+                                               c_int(_dt(proj, pool)), o._stream()), "window_kv_write")
+
+
 def pool_blocks(pool, cache_off: int, pool_off: int, kv_heads: int, dim: int, vdim: int, block_tables, row_seq,
                 positions, slots, block: int):
     """Pooled entries of a windowed attention that sees one mean key and value per block of ``block`` tokens
@@ -524,7 +542,7 @@ def window_decode_splits(rows: int, kv_heads: int, window: int, keep_first: int,
 def window_attention(q, pool, cache_off: int, kv_heads: int, vdim: int, block_tables, row_seq, positions, window: int,
                      keep_first: int, scale: float, softcap: float, sink, out=None, tiles=None, splits: int = 1,
                      own_values: bool = False, *, chunked: bool = False, pool_block: int = 0, pool_off: int = 0,
-                     maps: int = 1):
+                     maps: int = 1, head_gate=None):
     """Query rows q [T, heads, dim] over their sequences' cached keys: row i at position p sees key j when
     j <= p and (p - j < window or j < keep_first).  score = cap * tanh(q . k * scale / cap) (cap 0: none);
     softmax with ``sink`` [heads] (fp32, or None) in the denominator.  ``chunked``: ``window`` is a chunk size
@@ -539,7 +557,11 @@ def window_attention(q, pool, cache_off: int, kv_heads: int, vdim: int, block_ta
 
     bf16 rows of a shape the matrix-core kernel tiles take it: decode batches (``row_seq`` None) as they
     are (with ``splits`` key ranges per row, merged by a second launch), prefill rows when ``tiles`` (the
-    device copy of ``build_window_tiles``) describes them.  Everything else takes the plain kernel."""
+    device copy of ``build_window_tiles``) describes them.  Everything else takes the plain kernel.
+
+    ``head_gate`` [T, heads] (a view of a wider projection, activation dtype): a head's output is multiplied by the
+    sigmoid of its number.  ``out`` may be in the activation dtype instead of fp32 (what an output projection reads).
+    q's heads lie side by side; its rows may be those of a wider projection."""
     t, heads, dim = q.shape
     vsets = 1 if own_values else kv_heads
     if out is None:
@@ -551,28 +573,30 @@ def window_attention(q, pool, cache_off: int, kv_heads: int, vdim: int, block_ta
     if not q.is_cuda:
         return reference.window_attention(q, pool, cache_off, kv_heads, vdim, block_tables, row_seq, positions, window,
                                           keep_first, scale, softcap, sink, out, own_values, 1 if chunked else 0,
-                                          pool_block, pool_off, maps)
+                                          pool_block, pool_off, maps, head_gate)
     o = _ops()
-    _f32(sink, out)
+    _f32(sink)
     _i32(row_seq, positions)
-    assert q.is_contiguous() and block_tables.dtype == torch.int32 and block_tables.stride(1) == 1
+    assert out.dtype in (torch.float32, q.dtype) and out.is_contiguous() and out.numel() == t * heads * vsets * vdim
+    assert head_gate is None or (_rows(head_gate) and head_gate.shape == (t, heads) and head_gate.dtype == q.dtype)
+    assert q.stride(2) == 1 and (heads == 1 or q.stride(1) == dim) and block_tables.dtype == torch.int32 and block_tables.stride(1) == 1
     region = window_cache_elems(kv_heads, dim, vdim, kv_heads // maps)
     assert heads % kv_heads == 0 and cache_off + (pool_off if pool_block else 0) + region <= pool.shape[1]
     assert not pool_block or (pool_off >= region and (pool_off * pool.element_size()) % 16 == 0)
-    extra = (c_int(1 if chunked else 0), c_int(pool_block), c_long(pool_off), c_int(maps))
+    extra = (c_int(1 if chunked else 0), c_int(pool_block), c_long(pool_off), c_int(maps), o._p(head_gate),
+             c_long(head_gate.stride(0) if head_gate is not None else 0), c_int(1 if out.dtype != torch.float32 else 0))
     esz = pool.element_size()
     assert (cache_off * esz) % 16 == 0 and (pool.stride(0) * esz) % 16 == 0 and pool.data_ptr() % 16 == 0
     dt = _dt(q, pool)
     own = c_int(1 if own_values else 0)
     if (WINDOW_MFMA and dt == 0 and (tiles is not None or row_seq is None)
             and window_mfma_supported(heads, kv_heads, dim, vdim, own_values)
-            and q.data_ptr() % 16 == 0 and out.data_ptr() % 16 == 0):
+            and q.data_ptr() % 16 == 0 and q.stride(0) % 8 == 0 and out.data_ptr() % 16 == 0):
         ws_o = ws_ml = None
         if tiles is not None:
             assert tiles.dtype == torch.int32 and tiles.is_contiguous() and tiles.shape[1] == 4
             splits = 1
         elif splits > 1:
-            assert out.is_contiguous()
             ws_o = torch.empty((t * heads * splits * vsets * vdim,), dtype=torch.float32, device=q.device)
             ws_ml = torch.empty((t * heads * splits * 2,), dtype=torch.float32, device=q.device)
         o._check(o._kernels().vpsa_window_attention_mfma(
