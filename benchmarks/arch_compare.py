@@ -1,6 +1,6 @@
 """Prefill and decode throughput of one decoder design beside the closest existing one at equal size.
 
-    python bench.py --arch-compare zururax|revelix|pelatar|zetalorn|zupilorn [--arch-sizes s,m] [--arch-prompt 4096] [--arch-batch 32]
+    python bench.py --arch-compare zururax|revelix|pelatar|zetalorn|zupilorn|guzovik [--arch-sizes s,m] [--arch-prompt 4096] [--arch-batch 32]
 
 Random weights at layer shapes of real models (a few layers each); both models run through the same
 engine (scheduler, paged pool, HIP-graph decode).  Prefill: prompts of --arch-prompt tokens in chunks of
@@ -36,6 +36,8 @@ def _configs(design: str, size: str):
         return _zetalorn_configs(size)
     if design == "zupilorn":
         return _zupilorn_configs(size)
+    if design == "guzovik":
+        return _guzovik_configs(size)
     if design != "zururax":
         raise SystemExit(f"--arch-compare: unknown design {design!r}")
 
@@ -135,6 +137,21 @@ def _zupilorn_configs(size: str):
     new = zupilorn_config(f"zupilorn-{size}", VOCAB, z["width"],
                           zupilorn_stack(z["width"], z["heads"], ff, z["experts"], z["ff"], z["top"], blocks=z["layers"] // 2),
                           logit_softcap=30.0, max_position_embeddings=32768)
+    return new, _configs("zururax", size)[0]
+
+
+def _guzovik_configs(size: str):
+    """Guzovik (a sliding attention layer with a dense feed-forward, a sliding and a latent attention layer with routed
+    units and a shared one, and the second layer's tensors once more; windows of 1024 and 2048 positions) beside the
+    closest existing design, Zururax at the same width, depth, heads, latent rank, units, shared unit and dense
+    feed-forward: its latent attention runs the same kernels without a window, its units the same grouped GEMMs."""
+    from vllm_production_stack_amd.engine.config import guzovik_config, guzovik_stack
+
+    z = SIZES[size]
+    ff = z["top"] * z["ff"] + z["shared"]
+    new = guzovik_config(f"guzovik-{size}", VOCAB, z["width"],
+                         guzovik_stack(z["heads"], ff, z["experts"], z["ff"], z["top"], z["shared"]),
+                         embedding_scale=z["width"] ** 0.5, max_position_embeddings=32768)
     return new, _configs("zururax", size)[0]
 
 

@@ -415,10 +415,10 @@ def glu_act(x, act: str):
 
 def gate_up_act(x, w_gate_up, act: str, packed=None):
     """act(x @ Wg.T) * (x @ Wu.T) for ``w_gate_up = [Wg; Wu]``.  silu in bf16 is the fused path of the other
-    decoders (``gate_up_silu``); the tanh form of gelu runs in the prefill GEMM's epilogue when that kernel
+    decoders (``gate_up_silu``, units of a multiple of 8 channels); the tanh form of gelu runs in the prefill GEMM's epilogue when that kernel
     takes the shape; everything else is the projection and the activation kernel."""
     o = _ops()
-    if act == "silu" and x.is_cuda and x.dtype == torch.bfloat16:
+    if act == "silu" and x.is_cuda and x.dtype == torch.bfloat16 and w_gate_up.shape[0] % 16 == 0:
         return o.gate_up_silu(x, w_gate_up, packed)
     rows = o.tile_rows(x, w_gate_up, True) if (x.is_cuda and act == "gelu_tanh" and o.TILE_GELU_GLU) else 0
     if rows:
