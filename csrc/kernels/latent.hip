@@ -89,12 +89,23 @@ __device__ __forceinline__ void st8(bf16_t* p, const float* v) {
 __device__ __forceinline__ float sigmoidf(float x) { return 1.f / (1.f + expf(-x)); }
 
 // ---------------------------------------------------------------------------------
-template <typename T>
+// V: rows of whole runs of 8 values on 16-byte boundaries
+template <typename T, bool V>
 __global__ __launch_bounds__(256) void embed_scale_kernel(const long* __restrict__ ids, const T* __restrict__ embed,
                                                           float* __restrict__ out, int width, float scale) {
   const long row = blockIdx.x;
   const T* e = embed + ids[row] * (long)width;
   float* o = out + row * width;
+  if constexpr (V) {
+    for (int i = threadIdx.x * 8; i < width; i += 2048) {
+      float v[8];
+      ld8(e + i, v);
+#pragma unroll
+      for (int k = 0; k < 8; ++k) v[k] *= scale;
+      st8(o + i, v);
+    }
+    return;
+  }
   for (int i = threadIdx.x; i < width; i += 256) o[i] = Conv<T>::ld(e + i) * scale;
 }
 
@@ -466,21 +477,23 @@ __global__ __launch_bounds__(64) void route_softmax_kernel(const float* __restri
     c[e] = v + (bias ? bias[e] : 0.f);
   }
   __syncthreads();
-  const int per = n / groups;
-  for (int g = lane; g < groups; g += 64) {
-    float a = -INFINITY;
-    for (int e = g * per; e < (g + 1) * per; ++e) a = fmaxf(a, c[e]);
-    gs[g] = a;
+  if (keep < groups) {
+    const int per = n / groups;
+    for (int g = lane; g < groups; g += 64) {
+      float a = -INFINITY;
+      for (int e = g * per; e < (g + 1) * per; ++e) a = fmaxf(a, c[e]);
+      gs[g] = a;
+    }
+    __syncthreads();
+    for (int g = lane; g < groups; g += 64) {
+      int ahead = 0;
+      const float v = gs[g];
+      for (int o = 0; o < groups; ++o) ahead += (gs[o] > v) || (gs[o] == v && o < g);
+      if (ahead >= keep)
+        for (int e = g * per; e < (g + 1) * per; ++e) c[e] = -INFINITY;
+    }
+    __syncthreads();
   }
-  __syncthreads();
-  for (int g = lane; g < groups; g += 64) {
-    int ahead = 0;
-    const float v = gs[g];
-    for (int o = 0; o < groups; ++o) ahead += (gs[o] > v) || (gs[o] == v && o < g);
-    if (ahead >= keep)
-      for (int e = g * per; e < (g + 1) * per; ++e) c[e] = -INFINITY;
-  }
-  __syncthreads();
   float gsum = 0.f, wsum = 0.f;
   for (int k = 0; k < topk; ++k) {
     float best = -INFINITY;
@@ -968,9 +981,10 @@ inline int flat_grid(long total) {
 VPSA_EXPORT int vpsa_embed_scale(const long* ids, const void* embed, float* out, int rows, int width, float scale,
                                  int dtype, hipStream_t st) {
   if (rows <= 0) return 0;
-  DISPATCH(dtype,
-           hipLaunchKernelGGL(embed_scale_kernel<bf16_t>, dim3(rows), dim3(256), 0, st, ids, (const bf16_t*)embed, out, width, scale),
-           hipLaunchKernelGGL(embed_scale_kernel<float>, dim3(rows), dim3(256), 0, st, ids, (const float*)embed, out, width, scale));
+  const bool vec = width % 8 == 0 && (((uintptr_t)embed | (uintptr_t)out) & 15) == 0;
+#define ES(T, V) embed_scale_kernel<T, V><<<rows, 256, 0, st>>>(ids, (const T*)embed, out, width, scale)
+  DISPATCH(dtype, if (vec) ES(bf16_t, true); else ES(bf16_t, false), if (vec) ES(float, true); else ES(float, false));
+#undef ES
   return 0;
 }
 

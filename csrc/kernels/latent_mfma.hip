@@ -23,12 +23,17 @@
 // at the page of the first key that the tile's earliest query sees; only pages that hold a key some slot does not
 // see are masked key by key.
 //
-// Softmax state (running max, sum) is fp32 per slot; an optional per-head sink logit starts the state
+// Without q_lat (ROT_ONLY) the scores come from the entries' last ROT channels alone and the first RANK are values
+// only: the expanded per-head entries of a prefill, value | key.
+//
+// Softmax state (running max, sum) is fp32 per slot, scores in powers of two; an optional per-head sink logit starts the state
 // (max = sink, sum = 1).  With key-range splits every split writes unnormalised partial outputs and
 // (max, sum) to a workspace and a merge kernel adds the sink and normalises.
 #include "common.h"
 
 namespace {
+
+constexpr int MERGE_MAX = 64;  // key-range splits the merge kernel takes
 
 struct LatTile {
   int seq, row0, n_tok, pos0, head0, hcount;
@@ -36,17 +41,22 @@ struct LatTile {
 
 __device__ __forceinline__ u32x4 ld16(const uint16_t* p) { return *reinterpret_cast<const u32x4*>(p); }
 
-template <int RANK, int ROT>
-__global__ __launch_bounds__(256) void latent_mfma_kernel(
+constexpr float LOG2E = 1.4426950408889634f, LN2 = 0.6931471805599453f;
+
+// (entries of up to 256 values leave registers for three waves per SIMD; at 320 they would spill and lose)
+template <int RANK, int ROT, bool ROT_ONLY>
+__global__ __launch_bounds__(256, RANK + ROT <= 256 && RANK <= 128 ? 3 : 1) void latent_mfma_kernel(
     const uint16_t* __restrict__ q_lat, long ql_row, long ql_head, const uint16_t* __restrict__ q_rot, long qr_row,
     long qr_head, const uint16_t* __restrict__ cache, long page_stride, const int* __restrict__ block_tables,
     int bt_stride, const int* __restrict__ tiles, const int* __restrict__ positions, int heads,
     const float* __restrict__ sink, uint16_t* __restrict__ out, long o_row, long o_head, float scale, int window,
     int splits, float* __restrict__ ws_o, float* __restrict__ ws_ml) {
   constexpr int ENTRY = RANK + ROT;
-  constexpr int KS = ENTRY / 32;
+  constexpr int K0 = ROT_ONLY ? RANK : 0;     // first channel that scores read
+  constexpr int KC = ENTRY - K0;
+  constexpr int KS = KC / 32;
   constexpr int DT = RANK / 16;
-  constexpr int PK = ENTRY * 2 + 16;
+  constexpr int PK = KC * 2 + 16;
   constexpr int PV = 64 * 2 + 16;
   constexpr int NBLK = 2 * RANK;              // 4-key x 8-channel blocks of the latent part: 16 key quads x RANK / 8
   constexpr int RB = (NBLK + 255) / 256;      // of which a thread takes this many
@@ -70,6 +80,7 @@ __global__ __launch_bounds__(256) void latent_mfma_kernel(
   const int slot = wave * 16 + c16;
   const bool valid = slot < t.n_tok * t.hcount;
   const bool wave_active = wave * 16 < t.n_tok * t.hcount;  // wave-uniform
+  const float scale2 = scale * LOG2E;
   const int tok = valid ? slot / t.hcount : 0;
   const int head = t.head0 + (valid ? slot % t.hcount : 0);
   const long row = t.row0 + tok;
@@ -84,14 +95,14 @@ __global__ __launch_bounds__(256) void latent_mfma_kernel(
   bf16x8 qf[KS];
 #pragma unroll
   for (int ks = 0; ks < KS; ++ks) {
-    const int d = 32 * ks + 8 * g;
+    const int d = K0 + 32 * ks + 8 * g;
     u32x4 v = {0u, 0u, 0u, 0u};
     if (valid)
       v = d < RANK ? ld16(q_lat + row * ql_row + head * ql_head + d) : ld16(q_rot + row * qr_row + head * qr_head + (d - RANK));
     qf[ks] = __builtin_bit_cast(bf16x8, v);
   }
   const bool seeded = splits == 1 && sink != nullptr && valid;
-  float m = seeded ? sink[head] : -INFINITY;
+  float m = seeded ? sink[head] * LOG2E : -INFINITY;
   float l = seeded ? 1.f : 0.f;
   f32x4 o[DT];
 #pragma unroll
@@ -121,8 +132,10 @@ __global__ __launch_bounds__(256) void latent_mfma_kernel(
     for (int b = 0; b < RB; ++b) {
       const int id = tid + 256 * b, dc = id % (RANK / 8), kq = id / (RANK / 8);
       if (id >= NBLK) continue;
+      if constexpr (!ROT_ONLY) {
 #pragma unroll
-      for (int i = 0; i < 4; ++i) *reinterpret_cast<u32x4*>(kimg + (4 * kq + i) * PK + 16 * dc) = rb[b][i];
+        for (int i = 0; i < 4; ++i) *reinterpret_cast<u32x4*>(kimg + (4 * kq + i) * PK + 16 * dc) = rb[b][i];
+      }
       // keys 4 kq .. 4 kq + 3 = 16 n + 4 gg + e  ->  image position (n / 2) * 32 + gg * 8 + (n % 2) * 4 + e
       // = 16-byte chunk (n / 2) * 4 + gg, half n % 2.  Rows 8 dc .. 8 dc + 7 are written by one lane and
       // consecutive lanes hold consecutive dc, 8 rows = 1152 B apart: the chunk index is XORed with dc % 8
@@ -141,7 +154,7 @@ __global__ __launch_bounds__(256) void latent_mfma_kernel(
 #pragma unroll
     for (int b = 0; b < CB; ++b) {
       const int id = tid + 256 * b, dc = id % (ROT / 8), key = id / (ROT / 8);
-      *reinterpret_cast<u32x4*>(kimg + key * PK + 2 * RANK + 16 * dc) = cb[b];
+      *reinterpret_cast<u32x4*>(kimg + key * PK + 2 * (RANK - K0) + 16 * dc) = cb[b];
     }
   };
 
@@ -171,29 +184,35 @@ __global__ __launch_bounds__(256) void latent_mfma_kernel(
         const bf16x8 a = *reinterpret_cast<const bf16x8*>(kimg + (16 * nt + c16) * PK + (32 * ks + 8 * g) * 2);
         s[nt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, qf[ks], s[nt], 0, 0, 0);
       }
+#pragma unroll
+    for (int nt = 0; nt < 4; ++nt) s[nt] *= scale2;
+    // (where every slot of the tile sees the whole page there is nothing to mask)
+    if (p * PAGE + PAGE - 1 > t.pos0 || p * PAGE <= t.pos0 + t.n_tok - 1 - window) {
+#pragma unroll
+      for (int nt = 0; nt < 4; ++nt)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          const int key = p * PAGE + 16 * nt + 4 * g + e;
+          if (key > my_pos || key <= my_first) s[nt][e] = -INFINITY;
+        }
+    }
     float mx = -INFINITY;
-    // every slot of the tile sees the whole page: nothing to mask
-    const bool whole = p * PAGE + PAGE - 1 <= t.pos0 && p * PAGE > t.pos0 + t.n_tok - 1 - window;
 #pragma unroll
     for (int nt = 0; nt < 4; ++nt)
 #pragma unroll
-      for (int e = 0; e < 4; ++e) {
-        const int key = p * PAGE + 16 * nt + 4 * g + e;
-        const float v = whole || (key <= my_pos && key > my_first) ? s[nt][e] * scale : -INFINITY;
-        s[nt][e] = v;
-        mx = fmaxf(mx, v);
-      }
+      for (int e = 0; e < 4; ++e) mx = fmaxf(mx, s[nt][e]);
     mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
     mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
     const float mn = fmaxf(m, mx);
-    const bool dead = mn == -INFINITY;  // nothing seen so far and nothing visible here
-    const float corr = (dead || m == -INFINITY) ? (dead ? 1.f : 0.f) : __expf(m - mn);
+    const bool dead = mn == -INFINITY;   // nothing seen so far and nothing visible here:
+    const float mref = dead ? 0.f : mn;  // every score is -inf and weighs 0
+    const float corr = dead ? 1.f : __builtin_amdgcn_exp2f(m - mref);
     float ps = 0.f;
 #pragma unroll
     for (int nt = 0; nt < 4; ++nt)
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
-        const float pv = dead ? 0.f : __expf(s[nt][e] - mn);
+        const float pv = __builtin_amdgcn_exp2f(s[nt][e] - mref);
         s[nt][e] = pv;
         ps += pv;
       }
@@ -237,13 +256,15 @@ __global__ __launch_bounds__(256) void latent_mfma_kernel(
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) *reinterpret_cast<f32x4*>(dst + 16 * dt) = o[dt];
     if (g == 0) {
-      ws_ml[2 * rec] = m;
+      ws_ml[2 * rec] = m * LN2;
       ws_ml[2 * rec + 1] = l;
     }
   }
 }
 
-// One workgroup per (tile, slot): out = sum_s o_s exp(m_s - M) / (sum_s l_s exp(m_s - M) + exp(sink - M))
+// One workgroup per (tile, slot): out = sum_s o_s exp(m_s - M) / (sum_s l_s exp(m_s - M) + exp(sink - M)).  The splits'
+// factors are made once, by a wave with a split per lane; a thread then owns runs of 4 channels, all loads of a run in
+// flight together.
 __global__ __launch_bounds__(128) void latent_merge_kernel(const float* __restrict__ ws_o, const float* __restrict__ ws_ml,
                                                            const int* __restrict__ tiles, int heads,
                                                            const float* __restrict__ sink, uint16_t* __restrict__ out,
@@ -261,41 +282,53 @@ __global__ __launch_bounds__(128) void latent_merge_kernel(const float* __restri
   if (slot >= n_tok * hcount) return;
   const long row = row0 + slot / hcount;
   const int head = head0 + slot % hcount;
-  float big = sink ? sink[head] : -INFINITY;
-  for (int s = 0; s < splits; ++s) big = fmaxf(big, ws_ml[2 * (((long)tile * splits + s) * 64 + slot)]);
-  float den = sink ? __expf(sink[head] - big) : 0.f;
-  for (int s = 0; s < splits; ++s) {
-    const long rec = ((long)tile * splits + s) * 64 + slot;
-    const float ms = ws_ml[2 * rec];
-    if (ms != -INFINITY) den += ws_ml[2 * rec + 1] * __expf(ms - big);
+  __shared__ float fac[MERGE_MAX];  // 0: nothing was seen in the split (its record may hold anything)
+  const long rec0 = (long)tile * splits * 64 + slot;
+  if (threadIdx.x < 64) {
+    const int s = threadIdx.x;
+    const float ms = s < splits ? ws_ml[2 * (rec0 + 64L * s)] : -INFINITY;
+    const float ls = s < splits ? ws_ml[2 * (rec0 + 64L * s) + 1] : 0.f;
+    float big = wave_reduce_max(ms);
+    if (sink) big = fmaxf(big, sink[head]);
+    const float f = ms == -INFINITY ? 0.f : __expf(ms - big);
+    float den = wave_reduce_sum(f == 0.f ? 0.f : ls * f);
+    if (sink) den += __expf(sink[head] - big);
+    fac[s] = den > 0.f ? f / den : 0.f;
   }
-  const float inv = den > 0.f ? 1.f / den : 0.f;
-  for (int d = threadIdx.x; d < rank; d += 128) {
-    float a = 0.f;
-    for (int s = 0; s < splits; ++s) {
-      const long rec = ((long)tile * splits + s) * 64 + slot;
-      const float ms = ws_ml[2 * rec];
-      if (ms != -INFINITY) a += ws_o[rec * rank + d] * __expf(ms - big);
+  __syncthreads();
+  for (int d = threadIdx.x * 4; d < rank; d += 512) {
+    f32x4 a = {0.f, 0.f, 0.f, 0.f};
+    for (int s0 = 0; s0 < splits; s0 += 8) {
+      f32x4 v[8];
+#pragma unroll
+      for (int i = 0; i < 8; ++i)
+        v[i] = s0 + i < splits ? *reinterpret_cast<const f32x4*>(ws_o + (rec0 + 64L * (s0 + i)) * rank + d)
+                               : (f32x4){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int i = 0; i < 8; ++i) {
+        const float f = s0 + i < splits ? fac[s0 + i] : 0.f;
+        if (f != 0.f) a += v[i] * f;
+      }
     }
-    const bf16_t v = (bf16_t)(a * inv);
-    out[row * o_row + head * o_head + d] = __builtin_bit_cast(uint16_t, v);
+    u32x2 w = {pack_bf16x2(a[0], a[1]), pack_bf16x2(a[2], a[3])};
+    *reinterpret_cast<u32x2*>(out + row * o_row + head * o_head + d) = w;
   }
 }
 
-template <int RANK, int ROT>
+template <int RANK, int ROT, bool ROT_ONLY>
 int launch(const void* q_lat, long ql_row, long ql_head, const void* q_rot, long qr_row, long qr_head,
            const void* cache, long page_stride, const int* block_tables, int bt_stride, const int* tiles,
            const int* positions, int n_tiles, int heads, const float* sink, void* out, long o_row, long o_head,
            float scale, int window, int splits, float* ws_o, float* ws_ml, hipStream_t st) {
-  constexpr int LDS = 64 * ((RANK + ROT) * 2 + 16) + RANK * (64 * 2 + 16);
+  constexpr int LDS = 64 * ((ROT_ONLY ? ROT : RANK + ROT) * 2 + 16) + RANK * (64 * 2 + 16);
   static bool attr_set = false;
   if (!attr_set) {
-    if (hipFuncSetAttribute((const void*)latent_mfma_kernel<RANK, ROT>, hipFuncAttributeMaxDynamicSharedMemorySize,
+    if (hipFuncSetAttribute((const void*)latent_mfma_kernel<RANK, ROT, ROT_ONLY>, hipFuncAttributeMaxDynamicSharedMemorySize,
                             LDS) != hipSuccess)
       return -2;
     attr_set = true;
   }
-  latent_mfma_kernel<RANK, ROT><<<dim3(n_tiles, splits), dim3(256), LDS, st>>>(
+  latent_mfma_kernel<RANK, ROT, ROT_ONLY><<<dim3(n_tiles, splits), dim3(256), LDS, st>>>(
       (const uint16_t*)q_lat, ql_row, ql_head, (const uint16_t*)q_rot, qr_row, qr_head, (const uint16_t*)cache,
       page_stride, block_tables, bt_stride, tiles, positions, heads, sink, (uint16_t*)out, o_row, o_head, scale,
       window, splits, ws_o, ws_ml);
@@ -311,8 +344,8 @@ int launch(const void* q_lat, long ql_row, long ql_head, const void* q_rot, long
 // (latent entries: rank + rot; expanded per-head entries of a prefill: value | unrotated key | rotated key part,
 // rank = value channels, rot = the key's channels)
 #define LAT_SHAPES(X) \
-  X(64, 32) X(64, 64) X(128, 32) X(128, 64) X(256, 32) X(256, 64) X(512, 32) X(512, 64) \
-  X(32, 64) X(64, 96) X(64, 128) X(128, 128) X(128, 192)
+  X(64, 32) X(64, 64) X(128, 32) X(128, 64) X(256, 32) X(256, 64) X(512, 32) X(512, 64) LAT_EXPANDED(X)
+#define LAT_EXPANDED(X) X(32, 64) X(64, 96) X(64, 128) X(128, 128) X(128, 192)
 
 VPSA_EXPORT int vpsa_latent_mfma_supported(int rank, int rot) {
 #define LAT_IS(R, C) if (rank == R && rot == C) return 1;
@@ -321,10 +354,18 @@ VPSA_EXPORT int vpsa_latent_mfma_supported(int rank, int rot) {
   return 0;
 }
 
+// 1 when it also has the shape as value | key entries (no q_lat)
+VPSA_EXPORT int vpsa_latent_mfma_expanded(int rank, int rot) {
+#define LAT_IS(R, C) if (rank == R && rot == C) return 1;
+  LAT_EXPANDED(LAT_IS)
+#undef LAT_IS
+  return 0;
+}
+
 // tiles: int32 [n_tiles, 6] = (sequence, first query row, tokens, position of the first token, first head,
 // heads per token) with tokens * heads <= 64 and sequence < 0 for an unused entry; null = decode rows
 // (n_tiles = rows * ceil(heads / 64), positions [rows]).  Row and head strides in elements; every query
-// and output vector 16-byte / 8-byte aligned.  window >= 1 (a query sees itself and the window - 1 entries before
+// and output vector 16-byte / 8-byte aligned.  q_lat null: see ROT_ONLY above.  window >= 1 (a query sees itself and the window - 1 entries before
 // it; any window of at least the context length is plain causal attention).  splits > 1 needs ws_o [n_tiles * splits * 64 * rank] and
 // ws_ml [n_tiles * splits * 64 * 2] floats.
 VPSA_EXPORT int vpsa_latent_attention_mfma(const void* q_lat, long ql_row, long ql_head, const void* q_rot,
@@ -334,12 +375,20 @@ VPSA_EXPORT int vpsa_latent_attention_mfma(const void* q_lat, long ql_row, long 
                                            long o_row, long o_head, int rank, int rot, float scale, int window,
                                            int splits, float* ws_o, float* ws_ml, hipStream_t st) {
   if (n_tiles <= 0) return 0;
-  if (window < 1) return -1;
+  if (window < 1 || splits > MERGE_MAX) return -1;
   if (splits < 1 || splits > 65535 || (splits > 1 && (!ws_o || !ws_ml)) || (!tiles && !positions)) return -1;
   if (((ql_row | ql_head | qr_row | qr_head) & 7) || ((o_row | o_head) & 3) || (page_stride & 7)) return -1;
+#define LAT_ONLY(R, C)                                                                                              \
+  if (!q_lat && rank == R && rot == C)                                                                              \
+    return launch<R, C, true>(q_lat, ql_row, ql_head, q_rot, qr_row, qr_head, cache, page_stride, block_tables,      \
+                              bt_stride, tiles, positions, n_tiles, heads, sink, out, o_row, o_head, scale, window,   \
+                              splits, ws_o, ws_ml, st);
+  LAT_EXPANDED(LAT_ONLY)
+#undef LAT_ONLY
+  if (!q_lat) return -1;
 #define LAT_CASE(R, C)                                                                                              \
   if (rank == R && rot == C)                                                                                        \
-    return launch<R, C>(q_lat, ql_row, ql_head, q_rot, qr_row, qr_head, cache, page_stride, block_tables, bt_stride, \
+    return launch<R, C, false>(q_lat, ql_row, ql_head, q_rot, qr_row, qr_head, cache, page_stride, block_tables, bt_stride, \
                         tiles, positions, n_tiles, heads, sink, out, o_row, o_head, scale, window, splits, ws_o,      \
                         ws_ml, st);
   LAT_SHAPES(LAT_CASE)

@@ -528,14 +528,14 @@ __global__ __launch_bounds__(256) void qk_norm_write_kernel(const T* __restrict_
 // Keys and values of the step to the page layout of window_attention as they are (designs without norm or rotation,
 // whose queries the attention reads from the projection itself).  A workgroup takes 64 rows and 64 channels: keys are
 // copied row by row; values are turned through LDS, so that a channel's 64 tokens go out side by side (the rows of a
-// prompt's portion have neighbouring slots).  vec: key rows can be moved 16 bytes at a time.
+// prompt's portion have neighbouring slots).  vec / v_vec: key rows / value rows can be read 16 bytes at a time.
 constexpr int KVW = 64;
 
 template <typename T>
 __global__ __launch_bounds__(256) void window_kv_write_kernel(const T* __restrict__ k, const T* __restrict__ v,
                                                               long p_stride, const long* __restrict__ slots,
                                                               T* __restrict__ cache, long page_stride, int rows, int nk,
-                                                              int nv, int vec) {
+                                                              int nv, int vec, int v_vec) {
   constexpr int RUN = 16 / sizeof(T);
   __shared__ long base[KVW];  // where the row's token lies: its page's first element, and its place in the page
   __shared__ int place[KVW];
@@ -564,8 +564,19 @@ __global__ __launch_bounds__(256) void window_kv_write_kernel(const T* __restric
     return;
   }
   const int c0 = (blockIdx.y - k_blocks) * KVW, nc = min(KVW, nv - c0);
-  for (int r = wave; r < n; r += 4)
-    if (lane < nc) tile[r][lane] = v[(row0 + r) * p_stride + c0 + lane];
+  if (v_vec) {  // (nc is a multiple of RUN)
+    const int per = nc / RUN;
+    for (int i = tid; i < n * per; i += 256) {
+      const int r = i / per, c = i % per * RUN;
+      T x[RUN];
+      *reinterpret_cast<u32x4*>(x) = *reinterpret_cast<const u32x4*>(v + (row0 + r) * p_stride + c0 + c);
+#pragma unroll
+      for (int e = 0; e < RUN; ++e) tile[r][c + e] = x[e];
+    }
+  } else {
+    for (int r = wave; r < n; r += 4)
+      if (lane < nc) tile[r][lane] = v[(row0 + r) * p_stride + c0 + lane];
+  }
   __syncthreads();
   if (lane < n && base[lane] >= 0) {
     T* dst = cache + base[lane] + (long)PAGE * nk + place[lane];
@@ -840,6 +851,7 @@ __device__ __forceinline__ bool key_seen(int j, int p, int window, int keep_firs
 // out [rows, heads, kv_heads, vdim] fp32: the head's softmax weights applied to the values of every KV head
 // (the head mixing that follows needs them).  gate: the head's output times sigmoid(gate[row, head]); out_t: out is
 // in the activation dtype (what an output projection reads).
+constexpr float LOG2E = 1.4426950408889634f, LN2 = 0.6931471805599453f;
 constexpr int WA_KEYS = 256;
 constexpr int WA_ACC = 8;  // kv_heads * vdim <= 256 * WA_ACC
 
@@ -944,8 +956,10 @@ __global__ __launch_bounds__(256) void window_attention_kernel(
 // probabilities go from the first product's accumulators into the second without leaving the lane.
 // Scores are capped, masked by window / kept first tokens and normalised online in fp32; a sink logit starts
 // the running state (max = sink, sum = 1).  The next page's loads are in flight while a page is multiplied.
+// Up to 128 value channels the registers of three waves per SIMD are enough (512 TFLOP/s against 390 at 128 / 128
+// channels and the two waves that the compiler settles for by itself).
 template <int DIM, int VALL, int NSUB>
-__global__ __launch_bounds__(256) void window_mfma_kernel(
+__global__ __launch_bounds__(256, VALL <= 128 ? 3 : 1) void window_mfma_kernel(
     const uint16_t* __restrict__ q, long q_stride, const uint16_t* __restrict__ cache, long page_stride,
     const int* __restrict__ block_tables, int bt_stride, const int* __restrict__ tiles,
     const int* __restrict__ positions, const float* __restrict__ sink, void* __restrict__ out, int heads, int kv_heads,
@@ -1014,7 +1028,7 @@ __global__ __launch_bounds__(256) void window_mfma_kernel(
       qf[u][ks] = __builtin_bit_cast(bf16x8, v);
     }
     const bool seeded = splits == 1 && sink && valid[u];
-    m[u] = seeded ? sink[head[u]] : -INFINITY;
+    m[u] = seeded ? sink[head[u]] * LOG2E : -INFINITY;  // (scores and maxima in powers of two from here on)
     l[u] = seeded ? 1.f : 0.f;
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) o[u][dt] = (f32x4){0.f, 0.f, 0.f, 0.f};
@@ -1049,7 +1063,8 @@ __global__ __launch_bounds__(256) void window_mfma_kernel(
   int krow[4];
 #pragma unroll
   for (int nt = 0; nt < 4; ++nt) krow[nt] = (32 * (nt >> 1) + 8 * (c16 >> 2) + 4 * (nt & 1) + (c16 & 3)) * PK + 16 * g;
-  const float inv_cap = softcap > 0.f ? 1.f / softcap : 0.f;
+  const float inv_cap = softcap > 0.f ? scale / softcap : 0.f;
+  const float scale2 = scale * LOG2E, cap2 = softcap * LOG2E;
 
   if (i_begin < i_end) fetch(i_begin);
   for (int i = i_begin; i < i_end; ++i) {
@@ -1081,34 +1096,42 @@ __global__ __launch_bounds__(256) void window_mfma_kernel(
     float corr[NSUB];
 #pragma unroll
     for (int u = 0; u < NSUB; ++u) {
+      if (softcap > 0.f) {  // cap * tanh(v / cap), tanh(x) = 1 - 2 / (exp(2 x) + 1)
+#pragma unroll
+        for (int nt = 0; nt < 4; ++nt)
+#pragma unroll
+          for (int e = 0; e < 4; ++e)
+            s[u][nt][e] = cap2 * (1.f - 2.f / (__expf(2.f * inv_cap * s[u][nt][e]) + 1.f));
+      } else {
+#pragma unroll
+        for (int nt = 0; nt < 4; ++nt) s[u][nt] *= scale2;
+      }
+      if (!whole) {
+#pragma unroll
+        for (int nt = 0; nt < 4; ++nt)
+#pragma unroll
+          for (int e = 0; e < 4; ++e) {
+            const int j = j0 + 32 * (nt >> 1) + 8 * g + 4 * (nt & 1) + e;
+            if (!(pooled ? j < my_blocks[u] : key_seen(j, my_pos[u], window, keep_first, mode))) s[u][nt][e] = -INFINITY;
+          }
+      }
       float mx = -INFINITY;
 #pragma unroll
       for (int nt = 0; nt < 4; ++nt)
 #pragma unroll
-        for (int e = 0; e < 4; ++e) {
-          const int j = j0 + 32 * (nt >> 1) + 8 * g + 4 * (nt & 1) + e;
-          float v = -INFINITY;
-          if (whole || (pooled ? j < my_blocks[u] : key_seen(j, my_pos[u], window, keep_first, mode))) {
-            v = s[u][nt][e] * scale;
-            if (softcap > 0.f) {  // cap * tanh(v / cap), tanh(x) = 1 - 2 / (exp(2 x) + 1)
-              const float x = v * inv_cap;
-              v = softcap * (1.f - 2.f / (__expf(2.f * x) + 1.f));
-            }
-          }
-          s[u][nt][e] = v;
-          mx = fmaxf(mx, v);
-        }
+        for (int e = 0; e < 4; ++e) mx = fmaxf(mx, s[u][nt][e]);
       mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
       mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
       const float mn = fmaxf(m[u], mx);
-      const bool dead = mn == -INFINITY;
-      corr[u] = (dead || m[u] == -INFINITY) ? (dead ? 1.f : 0.f) : __expf(m[u] - mn);
+      const bool dead = mn == -INFINITY;       // nothing seen so far and nothing visible here:
+      const float mref = dead ? 0.f : mn;      // every score is -inf and weighs 0
+      corr[u] = dead ? 1.f : __builtin_amdgcn_exp2f(m[u] - mref);
       float psum = 0.f;
 #pragma unroll
       for (int nt = 0; nt < 4; ++nt)
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
-          const float pv = dead ? 0.f : __expf(s[u][nt][e] - mn);
+          const float pv = __builtin_amdgcn_exp2f(s[u][nt][e] - mref);
           s[u][nt][e] = pv;
           psum += pv;
         }
@@ -1165,7 +1188,7 @@ __global__ __launch_bounds__(256) void window_mfma_kernel(
 #pragma unroll
       for (int dt = 0; dt < DT; ++dt) *reinterpret_cast<f32x4*>(dst + 16 * dt) = o[u][dt];
       if (g == 0 && chunk == 0) {
-        ws_ml[2 * rec] = m[u];
+        ws_ml[2 * rec] = m[u] * LN2;
         ws_ml[2 * rec + 1] = l[u];
       }
     }
@@ -1679,9 +1702,10 @@ VPSA_EXPORT int vpsa_window_kv_write(const void* k, const void* v, long p_stride
   const int run = dt == 0 ? 8 : 4;
   const int vec = nk % run == 0 && p_stride % run == 0 && page_stride % run == 0 &&
                   (((uintptr_t)k | (uintptr_t)cache) & 15) == 0;
+  const int v_vec = nv % run == 0 && p_stride % run == 0 && ((uintptr_t)v & 15) == 0;
   const dim3 grid((rows + KVW - 1) / KVW, (nk + KVW - 1) / KVW + (nv + KVW - 1) / KVW);
   SM_DISPATCH(dt, (window_kv_write_kernel<T><<<grid, 256, 0, stream>>>((const T*)k, (const T*)v, p_stride, slots, (T*)cache,
-                                                                       page_stride, rows, nk, nv, vec)));
+                                                                       page_stride, rows, nk, nv, vec, v_vec)));
   return 0;
 }
 
@@ -1757,7 +1781,8 @@ VPSA_EXPORT int vpsa_window_mfma_supported(int heads, int kv_heads, int dim, int
 
 // Runs of 16 slots per wave in prefill tiles.  Two (a tile of 128 slots, every LDS fragment read half as often per
 // slot) need 256 accumulator registers per lane at 512 value channels; the compiler keeps them in the 256 arch
-// registers and spills (1.4 ms against 0.6 ms per 8192 rows), so one it is until the accumulators are placed by hand.
+// registers and spills (1.4 ms against 0.6 ms per 8192 rows).  At up to 128 channels, with registers for two waves per
+// SIMD, they were worth 5 % at 128 / 128 channels and lost 9 % at 64 / 64, beside one run and three waves per SIMD.
 #define WINDOW_PREFILL_SUB 1
 
 template <int DIM, int VALL, int NSUB>
@@ -1806,11 +1831,10 @@ VPSA_EXPORT int vpsa_window_attention_mfma(const void* q, long q_stride, const v
 #define WM(D, V)                                                                                                      \
   if (dim == D && vall == V) {                                                                                        \
     if (tiles)                                                                                                        \
-      return launch_window_mfma<D, V, WINDOW_PREFILL_SUB>(q, q_stride, cache, page_stride, block_tables, bt_stride,    \
-                                                          tiles, positions, sink, out, n_tiles, heads, kv_heads,      \
-                                                          window, keep_first, scale, softcap, splits, ws_o, ws_ml,     \
-                                                          n_chunks, own, mode, pool, pool_off, maps, gate, g_stride,  \
-                                                          out_t, stream);                                             \
+      return launch_window_mfma<D, V, WINDOW_PREFILL_SUB>(                                                             \
+          q, q_stride, cache, page_stride, block_tables, bt_stride, tiles, positions, sink, out, n_tiles, heads,      \
+          kv_heads, window, keep_first, scale, softcap, splits, ws_o, ws_ml, n_chunks, own, mode, pool, pool_off,     \
+          maps, gate, g_stride, out_t, stream);                                                                       \
     return launch_window_mfma<D, V, 1>(q, q_stride, cache, page_stride, block_tables, bt_stride, tiles, positions,     \
                                        sink, out, n_tiles, heads, kv_heads, window, keep_first, scale, softcap,       \
                                        splits, ws_o, ws_ml, n_chunks, own, mode, pool, pool_off, maps, gate,          \

@@ -279,6 +279,35 @@ def case_latent_window(dev, dtype, tol, shapes):
             attend(picks, row_seq, tiles=torch.from_numpy(ops.build_latent_tiles(q_lens, lens, heads)).to(dev))
 
 
+def case_expanded_entries(dev, shapes):
+    """Value | key entries of single heads on the tile kernel (bf16): scores from the key alone, windows, first tokens."""
+    dt = torch.bfloat16
+    g = torch.Generator().manual_seed(5)
+    for vdim, kdim, window in shapes:
+        heads, lens, q_lens = 2, [200, 70], [130, 70]
+        entry = vdim + kdim
+        pool, tables = paged(dev, dt, [n for n in lens for _ in range(heads)], PAGE * entry)
+        view = reference.latent_cache_view(pool, 0, entry)
+        q = torch.randn(sum(q_lens), heads, kdim, generator=g).to(dt)
+        want = torch.zeros(sum(q_lens), heads, vdim, dtype=F64)
+        tiles, row = [], 0
+        for i, (n, ctx) in enumerate(zip(q_lens, lens)):
+            seen = go.visible(ctx, window)[ctx - n:]
+            for h in range(heads):
+                e = (torch.randn(ctx, entry, generator=g) * 1.5).to(dt)
+                sl = slots_of(tables, i * heads + h, range(ctx))
+                view[(sl // PAGE).to(dev), (sl % PAGE).to(dev)] = e.to(dev)
+                sc = q[row:row + n, h].double() @ e[:, vdim:].double().T * 0.11
+                want[row:row + n, h] = go.weights_plain(sc, seen) @ e[:, :vdim].double()
+                tiles += [[i * heads + h, row + k, min(64, n - k), ctx - n + k, h, 1] for k in range(0, n, 64)]
+            row += n
+        pos = [p for n, ctx in zip(q_lens, lens) for p in range(ctx - n, ctx)]
+        out = torch.full((sum(q_lens), heads, vdim), float("nan"), dtype=dt, device=dev)
+        ops.latent_attention(None, q.to(dev), pool, 0, tables.to(dev), None, i32(pos, dev), None, 0.11, out=out,
+                             tiles=i32(tiles, dev), window=window)
+        close(out, want, 2e-2, f"{vdim} | {kdim}, window {window}")
+
+
 def case_routing(dev):
     """The softmax over the chosen logits alone, also where they are far from zero and far from each other."""
     g = torch.Generator().manual_seed(6)

@@ -67,6 +67,12 @@ def test_latent_window_on_the_matrix_cores(shape):
     gc.case_latent_window(DEV, "bfloat16", 2e-2, [shape])
 
 
+def test_expanded_entries():
+    shapes = [(32, 64, 50), (64, 96, 65), (64, 128, 1), (128, 128, 64), (128, 192, 1 << 30)]
+    assert all(ops.latent_expanded_supported(v, k) for v, k, _ in shapes)
+    gc.case_expanded_entries(DEV, shapes)
+
+
 @pytest.mark.parametrize("dtype", BOTH)
 def test_routing_mixture_and_clamped_unit(dtype):
     gc.case_routing(DEV)

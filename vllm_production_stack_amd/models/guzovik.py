@@ -60,7 +60,7 @@ class GuzovikModel(LatentAttention):
         self.max_model_len = max_model_len
         self.specs = cfg.layer_specs
         self.n_q = cfg.num_heads
-        self.n_kv = cfg.num_kv_heads
+        self.n_kv = 1   # (what the runner's split count of decode rows is for: the latent layers' shared entries)
         self.head_dim = cfg.head_dim
         self.tp_size = 1
         self.lora = None

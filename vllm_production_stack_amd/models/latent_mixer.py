@@ -53,7 +53,7 @@ class LatentAttention:
 
     def _expands(self, m: LatentMixerSpec) -> bool:
         return (self.device.type == "cuda" and self.dtype == torch.bfloat16 and m.kv_rank % 8 == 0 and m.rot_dim % 8 == 0
-                and ops.latent_mfma_supported(m.vdim, m.dim + m.rot_dim))
+                and ops.latent_expanded_supported(m.vdim, m.dim + m.rot_dim))
 
     # ------------------------------------------------------------------ batch description
     def plan_latent_prefill(self, meta: BatchMeta, q_lens: list[int], ctx_lens: list[int], to_dev, mixers) -> None:
@@ -103,9 +103,9 @@ class LatentAttention:
     def _expanded_prefill(self, lw, q: torch.Tensor, pool, meta: BatchMeta, plan: dict, out: torch.Tensor, offset: int):
         """Attention of the prefill rows with keys and values expanded per head for this step: the
         sequences' entries are gathered from the pool, one library product makes values and unrotated
-        keys of every head, and the tile kernel runs over per-head entries value | key | rotated part
-        (its first product reads zeros against the value channels).  640 / 2176 of the latent form's
-        FLOPs per query-key pair at 128 + 64 / 128 channels and rank 512."""
+        keys of every head, and the tile kernel runs over per-head entries value | unrotated key |
+        rotated part.  640 / 2176 of the latent form's FLOPs per query-key pair at 128 + 64 / 128 channels and rank
+        512."""
         m: LatentMixerSpec = lw.spec.mixer
         h, v, d, r, kr = m.heads, m.vdim, m.dim, m.rot_dim, m.kv_rank
         if lw.w_vk is None:
@@ -119,11 +119,7 @@ class LatentAttention:
             dst = exp[base:base + h * npg].view(h, npg, PAGE, wide)
             dst[:, :, :, :v + d] = vk.view(npg, PAGE, h, v + d).permute(2, 0, 1, 3)
             dst[:, :, :, v + d:] = ent[:, :, kr:].unsqueeze(0)
-        t = q.shape[0]
-        zeros = torch.zeros((1, 1, v), dtype=q.dtype, device=q.device).expand(t, h, v)
-        if not ops.latent_tile_kernel_takes(zeros, q, exp, out):
-            raise RuntimeError("expanded prefill: operands the tile kernel does not take")
-        ops.latent_attention(zeros, q, exp, 0, plan["bt"], None, meta.positions[meta.num_decode:], lw.sink, m.scale,
+        ops.latent_attention(None, q, exp, 0, plan["bt"], None, meta.positions[meta.num_decode:], lw.sink, m.scale,
                              out=out, tiles=plan["tiles"], window=m.window or NO_WINDOW)
 
     # ------------------------------------------------------------------ forward

@@ -39,7 +39,7 @@ def _kernels():
             "vpsa_tile_gemm", "vpsa_tile_gemm_debug", "vpsa_paged_prefill_split",
             "vpsa_embed_scale", "vpsa_add_rmsnorm", "vpsa_rmsnorm_rows", "vpsa_latent_kv_write", "vpsa_rope_pairs",
             "vpsa_latent_attention", "vpsa_sigmoid_gate", "vpsa_relu_sq", "vpsa_glu_clamp", "vpsa_group_topk",
-            "vpsa_gather_rows", "vpsa_moe_finish", "vpsa_latent_mfma_supported", "vpsa_latent_attention_mfma",
+            "vpsa_gather_rows", "vpsa_moe_finish", "vpsa_latent_mfma_supported", "vpsa_latent_mfma_expanded", "vpsa_latent_attention_mfma",
             "vpsa_moe_mfma_act",
             "vpsa_add_dyt", "vpsa_recurrent_scan", "vpsa_head_rms", "vpsa_short_conv_qkv", "vpsa_window_attention",
             "vpsa_mix_heads", "vpsa_xielu", "vpsa_window_mfma_supported", "vpsa_window_attention_mfma", "vpsa_window_tile_slots",
@@ -1353,7 +1353,7 @@ from .latent import (add_rms_norm, build_latent_tiles, embed_scale, gate_up_glu_
                      depth_mix_rms_norm, embed_rms_norm, moe_glu, poly_norm, soft_cap, up_poly_norm,
                      gate_up_act, gated_add_rms_norm, glu_act, rms_norm_add, route_softmax,
                      group_topk, latent_attention, moe_glu_grouped, moe_glu_grouped_supported, moe_units, moe_units_grouped, up_relu_sq,
-                     latent_kv_write, latent_mfma_supported, latent_tile_kernel_takes, moe_finish, relu_sq, rms_norm_rows, rope_pairs, sigmoid_gate)
+                     latent_expanded_supported, latent_kv_write, latent_mfma_supported, moe_finish, relu_sq, rms_norm_rows, rope_pairs, sigmoid_gate)
 
 # --------------------------------------------------------------------------- recurrent mixers, windowed attention, Dynamic Tanh
 from .seqmix import (add_dyt_norm, build_gru_pieces, build_scan_pieces, mingru_scan, build_window_tiles, head_rms_norm, mix_heads, recurrent_scan, short_conv_qkv,  # noqa: E402,F401

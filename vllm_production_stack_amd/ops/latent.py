@@ -264,20 +264,20 @@ def build_latent_tiles(q_lens, ctx_lens, heads: int):
     return tiles[order].astype(np.int32)
 
 
+def latent_expanded_supported(rank: int, rot: int) -> bool:
+    """Does the tile kernel take value | key entries of this shape (``latent_attention`` without ``q_lat``)?"""
+    return bool(_ops()._kernels().vpsa_latent_mfma_expanded(c_int(rank), c_int(rot)))
+
+
 def _mfma_ok(q_lat, q_rot, pool, out) -> bool:
-    if not (LATENT_MFMA and q_lat.dtype == torch.bfloat16 and pool.dtype == torch.bfloat16):
+    if not (LATENT_MFMA and q_rot.dtype == torch.bfloat16 and pool.dtype == torch.bfloat16):
         return False
-    rank, rot = q_lat.shape[2], q_rot.shape[2]
-    if not latent_mfma_supported(rank, rot):
+    rank, rot = out.shape[2], q_rot.shape[2]
+    if not (latent_mfma_supported(rank, rot) if q_lat is not None else latent_expanded_supported(rank, rot)):
         return False
-    return (q_lat.data_ptr() % 16 == 0 and q_rot.data_ptr() % 16 == 0 and out.data_ptr() % 8 == 0
-            and all(s % 8 == 0 for s in (q_lat.stride(0), q_lat.stride(1), q_rot.stride(0), q_rot.stride(1)))
-            and out.stride(0) % 4 == 0 and out.stride(1) % 4 == 0 and pool.stride(0) % 8 == 0)
-
-
-def latent_tile_kernel_takes(q_lat, q_rot, pool, out) -> bool:
-    """Would ``latent_attention`` run these operands on the matrix-core tile kernel?"""
-    return bool(q_lat.is_cuda and _mfma_ok(q_lat, q_rot, pool, out))
+    qs = [q for q in (q_lat, q_rot) if q is not None]
+    return (all(q.data_ptr() % 16 == 0 and q.stride(0) % 8 == 0 and q.stride(1) % 8 == 0 for q in qs)
+            and out.data_ptr() % 8 == 0 and out.stride(0) % 4 == 0 and out.stride(1) % 4 == 0 and pool.stride(0) % 8 == 0)
 
 
 def latent_attention(q_lat, q_rot, pool, offset: int, block_tables, row_seq, positions, sink, scale: float, out=None,
@@ -289,22 +289,28 @@ def latent_attention(q_lat, q_rot, pool, offset: int, block_tables, row_seq, pos
     ``block_tables[seq]`` and sees entries 0 .. positions[i], of these the last ``window``.  ``sink`` [heads] fp32 or None: a logit
     that joins the softmax denominator only.  Returns [T, heads, rank].
 
+    ``q_lat`` None (with ``out``, for shapes of ``latent_expanded_supported`` and rows that the tile kernel takes):
+    entries are value [rank] | key [rot] of one head, and the scores come from the key alone.
+
     bf16 entries of a shape the matrix-core kernel tiles take it: decode batches as they are (with
     ``splits`` key ranges per row, merged by a second launch), prefill rows when ``tiles`` (the device
     copy of ``build_latent_tiles``) describes them.  Everything else takes the plain kernel."""
-    t, heads, rank = q_lat.shape
+    t, heads = q_rot.shape[:2]
+    rank = q_lat.shape[2] if q_lat is not None else out.shape[2]
     assert 1 <= window <= NO_WINDOW
     if out is None:
-        out = torch.empty((t, heads, rank), dtype=q_lat.dtype, device=q_lat.device)
+        out = torch.empty((t, heads, rank), dtype=q_rot.dtype, device=q_rot.device)
     if t == 0:
         return out
-    if not q_lat.is_cuda:
+    if not q_rot.is_cuda:
         return reference.latent_attention(q_lat, q_rot, pool, offset, block_tables, row_seq, positions, sink, scale, out,
                                           window)
     o = _ops()
     rot = q_rot.shape[2]
     _f32(sink)
-    assert q_lat.stride(2) == 1 and q_rot.stride(2) == 1 and out.stride(2) == 1 and q_rot.shape[:2] == (t, heads)
+    assert q_rot.stride(2) == 1 and out.stride(2) == 1 and out.shape == (t, heads, rank)
+    assert q_lat is None or (q_lat.stride(2) == 1 and q_lat.shape[:2] == (t, heads))
+    ql_row, ql_head = (q_lat.stride(0), q_lat.stride(1)) if q_lat is not None else (0, 0)
     assert block_tables.dtype == torch.int32 and block_tables.stride(1) == 1 and positions.dtype == torch.int32
     assert row_seq is None or (row_seq.dtype == torch.int32 and row_seq.numel() == t)
     dt = _dt(q_lat, q_rot, pool, out)
@@ -319,14 +325,16 @@ def latent_attention(q_lat, q_rot, pool, offset: int, block_tables, row_seq, pos
             ws_o = torch.empty((n_tiles * splits * LATENT_TILE_SLOTS * rank,), dtype=torch.float32, device=out.device)
             ws_ml = torch.empty((n_tiles * splits * LATENT_TILE_SLOTS * 2,), dtype=torch.float32, device=out.device)
         o._check(o._kernels().vpsa_latent_attention_mfma(
-            o._p(q_lat), c_long(q_lat.stride(0)), c_long(q_lat.stride(1)), o._p(q_rot), c_long(q_rot.stride(0)),
+            o._p(q_lat), c_long(ql_row), c_long(ql_head), o._p(q_rot), c_long(q_rot.stride(0)),
             c_long(q_rot.stride(1)), _layer_base(pool, offset, rank + rot), c_long(pool.stride(0)), o._p(block_tables),
             c_int(block_tables.stride(0)), o._p(tiles), o._p(positions), c_int(n_tiles), c_int(heads), o._p(sink),
             o._p(out), c_long(out.stride(0)), c_long(out.stride(1)), c_int(rank), c_int(rot), c_float(scale),
             c_int(window), c_int(splits), o._p(ws_o), o._p(ws_ml), o._stream()), "latent_attention_mfma")
         return out
+    if q_lat is None:
+        raise ValueError("value | key entries: operands the tile kernel does not take")
     o._check(o._kernels().vpsa_latent_attention(
-        o._p(q_lat), c_long(q_lat.stride(0)), c_long(q_lat.stride(1)), o._p(q_rot), c_long(q_rot.stride(0)),
+        o._p(q_lat), c_long(ql_row), c_long(ql_head), o._p(q_rot), c_long(q_rot.stride(0)),
         c_long(q_rot.stride(1)), _layer_base(pool, offset, rank + rot), c_long(pool.stride(0)), o._p(block_tables),
         c_int(block_tables.stride(0)), o._p(row_seq), o._p(positions), o._p(sink), o._p(out), c_long(out.stride(0)),
         c_long(out.stride(1)), c_int(t), c_int(heads), c_int(rank), c_int(rot), c_float(scale),
