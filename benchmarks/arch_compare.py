@@ -4,7 +4,8 @@
 
 Random weights at layer shapes of real models (a few layers each); both models run through the same
 engine (scheduler, paged pool, HIP-graph decode).  Prefill: prompts of --arch-prompt tokens in chunks of
---max-num-batched-tokens, tokens per second until every prompt has its first token.  Decode:
+--max-num-batched-tokens, tokens per second until every prompt has its first token, the median of a few passes
+after one that is not timed.  Decode:
 --arch-batch sequences with --arch-context tokens of context each, tokens per second over the timed
 decode steps.  One JSON line per (size, model), then one summary line.
 """
@@ -22,6 +23,7 @@ SIZES = {
     "m": dict(width=4096, layers=4, heads=32, experts=32, ff=2048, top=4, shared=2048, q_rank=1536),
 }
 VOCAB = 32000
+PREFILL_PASSES = 5   # timed prefill passes (new prompts each), of which the median counts
 
 
 def _configs(design: str, size: str):
@@ -183,15 +185,18 @@ def _measure(cfg, a) -> dict:
 
     out = {"model": cfg.name, "params_b": round(cfg.num_params() / 1e9, 2)}
     # prefill
-    run_until_first_tokens(prompts(1, a.arch_prompt), 1)  # warm-up: library plans, lazy buffers
+    run_until_first_tokens(prompts(a.arch_prompts, a.arch_prompt), 1)  # warm-up: library plans, lazy buffers
     drain()
-    torch.cuda.synchronize()
-    t0 = time.perf_counter()
-    run_until_first_tokens(prompts(a.arch_prompts, a.arch_prompt), 1)
-    torch.cuda.synchronize()
-    dt = time.perf_counter() - t0
-    drain()
-    out["prefill_tok_s"] = round(a.arch_prompts * a.arch_prompt / dt, 1)
+    times = []
+    for _ in range(PREFILL_PASSES):
+        ps = prompts(a.arch_prompts, a.arch_prompt)
+        torch.cuda.synchronize()
+        t0 = time.perf_counter()
+        run_until_first_tokens(ps, 1)
+        torch.cuda.synchronize()
+        times.append(time.perf_counter() - t0)
+        drain()
+    out["prefill_tok_s"] = round(a.arch_prompts * a.arch_prompt / sorted(times)[PREFILL_PASSES // 2], 1)
     # decode
     reqs = run_until_first_tokens(prompts(a.arch_batch, a.arch_context), a.arch_decode_steps + 9)
     for _ in range(4):
